@@ -9,7 +9,8 @@
 // Math as in the reference's attention_block (crates/model/src/attention.rs:204-223) and its
 // decode kernel (crates/model/src/paged_attention.metal:56-198): query head h uses KV head
 // h / group; score = (q . k) * scale; a query at position p sees keys at positions <= p
-// (attention.rs:225-233) and, when a window w is given, > p - w; a position encoding that works
+// (attention.rs:225-233) and, when a window w is given, > p - w, or with chunks of c positions
+// those of its own chunk (floor(key / c) = floor(p / c)); a position encoding that works
 // on the scores gives `slopes` (one float per query head; the reference has none): the score of
 // key position u for a query at position p then gets slope * (u - p) added, in float32, before
 // the softmax; `head_scales` (one float per query head, or null) multiply the score scale of
@@ -34,7 +35,7 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(
     const int* __restrict__ block_tables, int max_pages, const int* __restrict__ seq_of_token,
     const int* __restrict__ positions, int nh, int nkv, int d, int page_size, float scale,
     int window, const float* __restrict__ slopes, const float* __restrict__ head_scales,
-    float softcap, const float* __restrict__ sinks, int keep_first) {
+    float softcap, const float* __restrict__ sinks, int keep_first, int chunk) {
   extern __shared__ float smem[];
   float* q_s = smem;                          // d
   float* p_s = smem + d;                      // 64
@@ -49,7 +50,7 @@ __global__ __launch_bounds__(64) void attn_generic_kernel(
   const float inv_cap = softcap > 0.f ? 1.0f / softcap : 0.f;
   for (int j = lane; j < d; j += 64) q_s[j] = ld(q + (long long)t * q_stride + h * d + j) * scale;
   __syncthreads();
-  const int lo = (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+  const int lo = first_visible(pos, window, chunk);
   float m = -INFINITY, l = 0.f;
   float acc[DPL];
 #pragma unroll
@@ -119,8 +120,10 @@ RLIS_API int rlis_attn_generic(const void* q, int dtype, long long q_stride, voi
                                const int* positions, int T, int nh, int nkv, int d, int page_size,
                                float scale, int window, const float* slopes,
                                const float* head_scales, float softcap, const float* sinks,
-                               int keep_first, hipStream_t stream) {
+                               int keep_first, int chunk, hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && nh > 0 && nkv > 0 && d > 0 && page_size > 0, "attn_generic: bad sizes");
+  RLIS_REQUIRE(chunk >= 0 && (chunk == 0 || (window == 0 && keep_first == 0)),
+               "attn_generic: a window or chunks, not both");
   RLIS_REQUIRE(keep_first >= 0, "attn_generic: bad count of kept first keys");
   RLIS_REQUIRE(nh % nkv == 0, "attn_generic: %d query heads are not a multiple of %d KV heads",
                nh, nkv);
@@ -134,7 +137,7 @@ RLIS_API int rlis_attn_generic(const void* q, int dtype, long long q_stride, voi
   attn_generic_kernel<TX, DPL><<<grid, 64, smem, stream>>>(                                    \
       (const TX*)q, q_stride, (TX*)out, out_stride, (const TX*)k_pages, (const TX*)v_pages,    \
       block_tables, max_pages, seq_of_token, positions, nh, nkv, d, page_size, scale, window,  \
-      slopes, head_scales, softcap, sinks, keep_first)
+      slopes, head_scales, softcap, sinks, keep_first, chunk)
 #define BY_DPL(TX)                         \
   do {                                     \
     if (dpl <= 1) LAUNCH(TX, 1);           \
@@ -190,7 +193,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
     const int* __restrict__ ctx_lens, const int* __restrict__ token_rows, int nh, int nkv, int d,
     int page_size, float scale, int window, int splits, int chunks_per_kv, int part_keys,
     int max_parts, const float* __restrict__ slopes, const float* __restrict__ head_scales,
-    float softcap, const float* __restrict__ sinks, int keep_first) {
+    float softcap, const float* __restrict__ sinks, int keep_first, int chunk_len) {
   extern __shared__ float smem[];
   float* q_s = smem;                     // G * d
   float* p_s = q_s + G * d;              // 4 waves * G * 64
@@ -206,7 +209,7 @@ __global__ __launch_bounds__(256) void attn_decode_kernel(
   const int ctx = ctx_lens[seq];
   const int row = token_rows ? token_rows[seq] : seq;
   const int* table = block_tables + (long long)seq * max_pages;
-  const int lo = (window > 0 && ctx - window > 0) ? ctx - window : 0;
+  const int lo = first_visible(ctx - 1, window, chunk_len);
   const int nkeys = ctx - lo;
   const int part = decode_part_len(nkeys, part_keys, max_parts);
   const int kbeg = lo + split * part;
@@ -551,7 +554,8 @@ static int launch_decode(const void* q, long long q_stride, void* out, long long
                          const int* ctx_lens, const int* token_rows, int S, int nh, int nkv, int d,
                          int page_size, float scale, int window, int splits, int part_keys,
                          int max_parts, const float* slopes, const float* head_scales,
-                         float softcap, const float* sinks, int keep_first, hipStream_t stream) {
+                         float softcap, const float* sinks, int keep_first, int chunk_len,
+                         hipStream_t stream) {
   const int g = nh / nkv;
   const int chunks = ceil_div(g, G);
   dim3 grid(nkv * chunks, S, splits);
@@ -564,7 +568,7 @@ static int launch_decode(const void* q, long long q_stride, void* out, long long
       (const TX*)q, q_stride, (TX*)out, out_stride, part_ml, part_acc, (const TX*)k_pages,     \
       (const TX*)v_pages, block_tables, max_pages, ctx_lens, token_rows, nh, nkv, d, page_size, \
       scale, window, splits, chunks, part_keys, max_parts, slopes, head_scales, softcap,       \
-      sinks, keep_first)
+      sinks, keep_first, chunk_len)
   if (dpl <= 1) LAUNCH(1);
   else if (dpl <= 2) LAUNCH(2);
   else LAUNCH(4);
@@ -584,8 +588,10 @@ RLIS_API int rlis_attn_decode(const void* q, int dtype, long long q_stride, void
                               int nh, int nkv, int d, int page_size, float scale, int window,
                               int splits, int part_keys, int max_parts, const float* slopes,
                               const float* head_scales, float softcap, const float* sinks,
-                              int keep_first, hipStream_t stream) {
+                              int keep_first, int chunk, hipStream_t stream) {
   RLIS_REQUIRE(S >= 0 && nh > 0 && nkv > 0 && d > 0 && page_size > 0, "attn_decode: bad sizes");
+  RLIS_REQUIRE(chunk >= 0 && (chunk == 0 || (window == 0 && keep_first == 0)),
+               "attn_decode: a window or chunks, not both");
   RLIS_REQUIRE(part_keys >= 64 && part_keys % 64 == 0 && max_parts >= 1 && splits <= max_parts,
                "attn_decode: partitions of %d keys (a multiple of 64), %d deep of at most %d",
                part_keys, splits, max_parts);
@@ -604,22 +610,22 @@ RLIS_API int rlis_attn_decode(const void* q, int dtype, long long q_stride, void
       rc = launch_decode<TX, 1>(q, q_stride, out, out_stride, part_ml, part_acc, k_pages,        \
                                 v_pages, block_tables, max_pages, ctx_lens, token_rows, S, nh,   \
                                 nkv, d, page_size, scale, window, splits, part_keys, max_parts,       \
-                                slopes, head_scales, softcap, sinks, keep_first, stream); \
+                                slopes, head_scales, softcap, sinks, keep_first, chunk, stream); \
     else if (g == 2)                                                                             \
       rc = launch_decode<TX, 2>(q, q_stride, out, out_stride, part_ml, part_acc, k_pages,        \
                                 v_pages, block_tables, max_pages, ctx_lens, token_rows, S, nh,   \
                                 nkv, d, page_size, scale, window, splits, part_keys, max_parts,       \
-                                slopes, head_scales, softcap, sinks, keep_first, stream); \
+                                slopes, head_scales, softcap, sinks, keep_first, chunk, stream); \
     else if (g <= 4)                                                                             \
       rc = launch_decode<TX, 4>(q, q_stride, out, out_stride, part_ml, part_acc, k_pages,        \
                                 v_pages, block_tables, max_pages, ctx_lens, token_rows, S, nh,   \
                                 nkv, d, page_size, scale, window, splits, part_keys, max_parts,       \
-                                slopes, head_scales, softcap, sinks, keep_first, stream); \
+                                slopes, head_scales, softcap, sinks, keep_first, chunk, stream); \
     else                                                                                         \
       rc = launch_decode<TX, 8>(q, q_stride, out, out_stride, part_ml, part_acc, k_pages,        \
                                 v_pages, block_tables, max_pages, ctx_lens, token_rows, S, nh,   \
                                 nkv, d, page_size, scale, window, splits, part_keys, max_parts,       \
-                                slopes, head_scales, softcap, sinks, keep_first, stream); \
+                                slopes, head_scales, softcap, sinks, keep_first, chunk, stream); \
   } while (0)
   if (dtype == RLIS_F32) BY_G(float);
   else if (dtype == RLIS_BF16) BY_G(bf16_t);

@@ -22,7 +22,8 @@
 //
 // The mask is the reference's causal mask offset by the cached length (crates/model/src/
 // attention.rs:225-233): the new token at index i of a sequence with P cached positions sees
-// keys at positions <= P + i, and > P + i - window when a window is given.  Scores are scaled
+// keys at positions <= P + i, and > P + i - window when a window is given, or those of its own
+// chunk of positions when chunks are.  Scores are scaled
 // in float32 after the product (kept in the base-2 domain so that e^x is one v_exp_f32);
 // probabilities are rounded to bfloat16 only as the operand of the second product (the row
 // sums use the float32 values).
@@ -119,7 +120,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((QB == 1 &&
     int row0, float* __restrict__ part_ml, float* __restrict__ part_acc,
     const float* __restrict__ cos_t, const float* __restrict__ sin_t,
     const float* __restrict__ slopes, const float* __restrict__ head_scales, float softcap,
-    const float* __restrict__ sinks, int keep_first) {
+    const float* __restrict__ sinks, int keep_first, int chunk) {
   constexpr int BN = tile_keys(QB);
   // V^T tile rows: 64 keys padded to a stride of 32 bytes mod 64; 32 keys unpadded, with the
   // 16-byte piece index XORed with (-(row / 4)) & 3, which frees reads and stores of conflicts.
@@ -210,8 +211,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((QB == 1 &&
 
   const int q_last = min(n_new, qb + BM * QB) - 1;      // last new-token index of the tile
   const int khi_all = P + q_last + 1;                    // keys [klo, khi_all) matter to the tile
-  int klo = 0;
-  if (window > 0) klo = max(0, P + qb - window + 1);
+  const int klo = first_visible(P + qb, window, chunk);
   int kt0_all = (klo / BN) * BN;
   // With first keys of the sequence that stay visible in front of the window, the tile walks
   // two runs of key tiles: those that hold kept keys, [0, kept_end), and the window's from
@@ -238,6 +238,12 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((QB == 1 &&
     khi = min(khi_walk, kt0 + per * BN);
   }
   const int wave_q_last = min(n_new - 1, wave_q_first + 16 * QB - 1);
+  // the first key each of this lane's queries sees, and the first that all of the wave's see
+  // (what a query sees never starts earlier than what the query before it does)
+  int my_lo[QB];
+#pragma unroll
+  for (int b = 0; b < QB; ++b) my_lo[b] = first_visible(my_qpos[b], window, chunk);
+  const int wave_lo = first_visible(P + wave_q_first + 16 * QB - 1, window, chunk);
 
   // Staging for the tiles to come.  A tile's page ids are fetched four tiles ahead of its use,
   // its keys and values two tiles ahead (two register sets taking turns), so that neither the
@@ -402,8 +408,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((QB == 1 &&
       }
       // ---- scale, mask (only where a tile meets the diagonal, the window or the end) -----
       const bool plain_tile = (k0 + BN - 1 <= P + wave_q_first) &&
-                              (window <= 0 || k0 > P + wave_q_first + 16 * QB - 1 - window ||
-                               k0 + BN <= keep_first);
+                              (k0 >= wave_lo || k0 + BN <= keep_first);
       // The scale (positive) is applied inside the exponent, with one fused multiply-add per
       // score; the maximum is taken over the raw scores and scaled once.
       bool moved = false;
@@ -423,7 +428,7 @@ __global__ __launch_bounds__(256) __attribute__((amdgpu_waves_per_eu((QB == 1 &&
             for (int r = 0; r < 4; ++r) {
               const int kpos = k0 + (nb / 2) * 32 + lq * 8 + 2 * r + (nb % 2);
               const bool ok = (kpos <= my_qpos[b]) &&
-                              (window <= 0 || kpos > my_qpos[b] - window || kpos < keep_first);
+                              (kpos >= my_lo[b] || kpos < keep_first);
               const float sv = ok ? s[b][nb][r] : -INFINITY;
               s[b][nb][r] = sv;
               mx = fmaxf(mx, sv);
@@ -580,7 +585,7 @@ RLIS_API int RLIS_CAT(rlis_attn_prefill_mfma_d, RLIS_HEAD_DIM)(
     int page_shift, int window, float scale, int tile_queries, int splits, int row0,
     float* part_ml, float* part_acc, const float* cos, const float* sin, int rot,
     const float* slopes, const float* head_scales, float softcap, const float* sinks,
-    int keep_first, hipStream_t stream) {
+    int keep_first, int chunk, hipStream_t stream) {
   if (num_tiles == 0) return 0;
   const bool shaped = slopes || head_scales || softcap > 0.f;
   // rotation inside the kernel needs head_dim = rotated width = 64, 128 or 256
@@ -594,7 +599,7 @@ RLIS_API int RLIS_CAT(rlis_attn_prefill_mfma_d, RLIS_HEAD_DIM)(
       (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, (const bf16_t*)k_pages,              \
       (const bf16_t*)v_pages, block_tables, max_pages, cu_seqlens, start_pos, tile_map, nh, nkv, \
       d, page_shift, scale, window, num_tiles, tiles_per_round, splits, row0, part_ml, part_acc, \
-      cos, sin, slopes, head_scales, softcap, sinks, keep_first)
+      cos, sin, slopes, head_scales, softcap, sinks, keep_first, chunk)
   if (tile_queries == 2 * BM) {
     if (shaped) RLIS_PREFILL_LAUNCH(2, true);
     else RLIS_PREFILL_LAUNCH(2, false);
@@ -701,8 +706,9 @@ __global__ __launch_bounds__(512, RLIS_HEAD_DIM <= 64 ? 4 : 2) void DECODE_KERNE
     int max_parts, int merge_inside, int groups, int cap, const DecodeRope rope,
     const DecodeMerge merge, const float* __restrict__ slopes,
     const float* __restrict__ head_scales, float softcap, const float* __restrict__ sinks,
-    int keep_first) {
+    int keep_first, int chunk_len) {
   if constexpr (EXACT) {
+    chunk_len = 0;
     d = D;
     page_shift = kExactPageShift;
     window = 0;
@@ -749,7 +755,7 @@ __global__ __launch_bounds__(512, RLIS_HEAD_DIM <= 64 ? 4 : 2) void DECODE_KERNE
   // ---- what follows from the context length ---------------------------------------------
   const int* table = block_tables + (long long)seq * max_pages;
   const int page_mask = (1 << page_shift) - 1;
-  const int lo = (window > 0 && ctx - window > 0) ? ctx - window : 0;
+  const int lo = first_visible(ctx - 1, window, chunk_len);
   int lo32 = lo & ~31;
   // With first keys of the sequence that stay visible in front of the window, the keys walked
   // are two runs: the chunks that hold kept keys, [0, kept32), and the window's from lo32 on.
@@ -1186,7 +1192,7 @@ RLIS_API int RLIS_CAT(rlis_attn_decode_mfma_d, RLIS_HEAD_DIM)(
     int max_pages, const int* ctx_lens, int S, int nh, int nkv, int d, int page_shift, int window,
     float scale, int splits, int part_keys, int max_parts, int merge_inside, int groups, int cap,
     const DecodeRope* rope, const DecodeMerge* merge, const float* slopes,
-    const float* head_scales, float softcap, const float* sinks, int keep_first,
+    const float* head_scales, float softcap, const float* sinks, int keep_first, int chunk,
     hipStream_t stream) {
   if (S == 0) return 0;
   const bool shaped = slopes || head_scales || softcap > 0.f;
@@ -1231,8 +1237,8 @@ RLIS_API int RLIS_CAT(rlis_attn_decode_mfma_d, RLIS_HEAD_DIM)(
       (const bf16_t*)q, q_stride, (bf16_t*)out, out_stride, part_ml, part_acc,                   \
       (const bf16_t*)k_pages, (const bf16_t*)v_pages, block_tables, max_pages, ctx_lens, nh, nkv, \
       d, page_shift, scale, window, splits, part_keys, max_parts, merge_inside, groups, cap,   \
-      *rope, *merge, slopes, head_scales, softcap, sinks, keep_first)
-  const bool exact = d == D && page_shift == kExactPageShift && window <= 0;
+      *rope, *merge, slopes, head_scales, softcap, sinks, keep_first, chunk)
+  const bool exact = d == D && page_shift == kExactPageShift && window <= 0 && chunk == 0;
   if (shaped && cap > 1) RLIS_DEC_LAUNCH(true, false, true);
   else if (shaped) RLIS_DEC_LAUNCH(false, false, true);
   else if (cap > 1 && exact) RLIS_DEC_LAUNCH(true, true, false);

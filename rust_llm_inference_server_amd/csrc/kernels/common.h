@@ -35,6 +35,23 @@ __device__ __forceinline__ float widen(bf16_t v) { return bf16_to_f32(v); }
 __device__ __forceinline__ void st(float* p, float v) { *p = v; }
 __device__ __forceinline__ void st(bf16_t* p, float v) { *p = f32_to_bf16(v); }
 
+// The tanh form of GELU, float32: 0.5 x (1 + tanh z), z = sqrt(2 / pi) (x + 0.044715 x^3), and
+// 2 z / x, for the forms that take 0.5 (1 + tanh z) as the sigmoid of 2 z.
+__device__ __forceinline__ float gelu_tanh_f(float x) {
+  const float inner = 0.7978845608028654f * (x + 0.044715f * x * x * x);
+  return 0.5f * x * (1.0f + tanhf(inner));
+}
+__device__ __forceinline__ float gelu_slope(float x) {
+  return 1.5957691216057308f * (1.0f + 0.044715f * x * x);
+}
+
+// The first key position that a query at `pos` sees: all (0), a sliding window's, or the start
+// of its own chunk of positions (window and chunk 0: none; never both).
+__device__ __forceinline__ int first_visible(int pos, int window, int chunk) {
+  if (chunk > 0) return pos - pos % chunk;
+  return (window > 0 && pos - window + 1 > 0) ? pos - window + 1 : 0;
+}
+
 // A delta for the residual stream that arrives as `parts` float32 partial sums, part_stride
 // elements apart: they are added in order and, with round16, the sum is rounded to bfloat16 as
 // a delta that arrives whole in bfloat16 was, so that a block's output is rounded once to the

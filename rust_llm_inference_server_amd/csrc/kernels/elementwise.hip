@@ -438,8 +438,9 @@ RLIS_API int rlis_add_rmsnorm(float* resid, const void* delta, int delta_dtype,
 }
 
 // -------------------------------------------------------------------------- SwiGLU
-// gu (T, 2I): columns [0, I) are the gate projection, [I, 2I) the up projection.
-template <typename TX>
+// gu (T, 2I): columns [0, I) are the gate projection, [I, 2I) the up projection.  GELU: the gate
+// passes the tanh form of GELU instead of SiLU.
+template <typename TX, bool GELU>
 __global__ void swiglu_kernel(TX* __restrict__ out, const TX* __restrict__ gu, int I,
                               long long total) {
   long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
@@ -449,12 +450,13 @@ __global__ void swiglu_kernel(TX* __restrict__ out, const TX* __restrict__ gu, i
     const int c = (int)(i - t * I);
     const float g = ld(gu + t * 2 * I + c);
     const float u = ld(gu + t * 2 * I + I + c);
-    const float s = g / (1.0f + expf(-g));
+    const float s = GELU ? gelu_tanh_f(g) : g / (1.0f + expf(-g));
     st(out + i, s * u);
   }
 }
 
 // bfloat16 rows whose width is a multiple of 8: eight columns per thread, 16-byte accesses.
+template <bool GELU>
 __global__ void swiglu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* __restrict__ gu,
                                      int I8 /* I / 8 */, long long total8) {
   long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
@@ -473,8 +475,10 @@ __global__ void swiglu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* __r
       // silu(g) * u with the hardware's exponential and reciprocal (an ulp each, far inside
       // what the rounding to bfloat16 leaves): the library functions made this kernel spend as
       // long on arithmetic as on its bytes.
-      const float e0 = __builtin_amdgcn_exp2f(g0 * -1.4426950408889634f);
-      const float e1 = __builtin_amdgcn_exp2f(g1 * -1.4426950408889634f);
+      // (GELU's 0.5 (1 + tanh z) is sigmoid(2 z), z = sqrt(2 / pi) (g + 0.044715 g^3))
+      const float a0 = GELU ? gelu_slope(g0) * g0 : g0, a1 = GELU ? gelu_slope(g1) * g1 : g1;
+      const float e0 = __builtin_amdgcn_exp2f(a0 * -1.4426950408889634f);
+      const float e1 = __builtin_amdgcn_exp2f(a1 * -1.4426950408889634f);
       const float r0 = g0 * __builtin_amdgcn_rcpf(1.0f + e0) * u0;
       const float r1 = g1 * __builtin_amdgcn_rcpf(1.0f + e1) * u1;
       ow[j] = (uint32_t)f32_to_bf16(r0) | ((uint32_t)f32_to_bf16(r1) << 16);
@@ -483,26 +487,35 @@ __global__ void swiglu_bf16x8_kernel(bf16_t* __restrict__ out, const bf16_t* __r
   }
 }
 
-RLIS_API int rlis_swiglu(void* out, const void* gu, int dtype, int T, int I, hipStream_t stream) {
+template <bool GELU>
+static int launch_swiglu(void* out, const void* gu, int dtype, int T, int I, hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && I > 0, "swiglu: bad sizes T=%d I=%d", T, I);
   const long long total = (long long)T * I;
   if (total == 0) return 0;
   if (dtype == RLIS_BF16 && I % 8 == 0 && ((uintptr_t)out % 16) == 0 && ((uintptr_t)gu % 16) == 0) {
     const long long total8 = total / 8;
     const int blocks8 = (int)(ceil_div_ll(total8, 256) < 16384 ? ceil_div_ll(total8, 256) : 16384);
-    swiglu_bf16x8_kernel<<<blocks8, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)gu, I / 8, total8);
+    swiglu_bf16x8_kernel<GELU><<<blocks8, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)gu, I / 8, total8);
     RLIS_LAUNCH_CHECK("swiglu");
     return 0;
   }
   const int blocks = (int)(ceil_div_ll(total, 256) < 8192 ? ceil_div_ll(total, 256) : 8192);
   if (dtype == RLIS_F32)
-    swiglu_kernel<float><<<blocks, 256, 0, stream>>>((float*)out, (const float*)gu, I, total);
+    swiglu_kernel<float, GELU><<<blocks, 256, 0, stream>>>((float*)out, (const float*)gu, I, total);
   else if (dtype == RLIS_BF16)
-    swiglu_kernel<bf16_t><<<blocks, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)gu, I, total);
+    swiglu_kernel<bf16_t, GELU><<<blocks, 256, 0, stream>>>((bf16_t*)out, (const bf16_t*)gu, I, total);
   else
     RLIS_REQUIRE(false, "swiglu: unknown dtype %d", dtype);
   RLIS_LAUNCH_CHECK("swiglu");
   return 0;
+}
+
+RLIS_API int rlis_swiglu(void* out, const void* gu, int dtype, int T, int I, hipStream_t stream) {
+  return launch_swiglu<false>(out, gu, dtype, T, I, stream);
+}
+
+RLIS_API int rlis_geglu(void* out, const void* gu, int dtype, int T, int I, hipStream_t stream) {
+  return launch_swiglu<true>(out, gu, dtype, T, I, stream);
 }
 
 // ------------------------------------------------------------- clamped gated unit
@@ -627,10 +640,6 @@ RLIS_API int rlis_weighted_sum(float* out, const void* x, int x_dtype, float a, 
 
 // ------------------------------------------------------------- tanh form of GELU
 // y = 0.5 x (1 + tanh(sqrt(2 / pi) (x + 0.044715 x^3))), float32 arithmetic, one rounding.
-__device__ __forceinline__ float gelu_tanh_f(float x) {
-  const float inner = 0.7978845608028654f * (x + 0.044715f * x * x * x);
-  return 0.5f * x * (1.0f + tanhf(inner));
-}
 
 template <typename TX>
 __global__ void gelu_tanh_kernel(TX* __restrict__ out, const TX* __restrict__ x, long long n) {

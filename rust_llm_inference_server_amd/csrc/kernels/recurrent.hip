@@ -14,15 +14,11 @@
 // a sum over the wave, and nothing is shared between waves, so the columns of a head spread
 // over the chip.  State layout per head: [value channel][key channel], so a wave's columns are
 // contiguous.
-#include "common.h"
+#include "scan.h"
 
 namespace {
 
 constexpr int kMaxTaps = 16;
-
-__device__ __forceinline__ float sigmoidf_(float x) { return 1.0f / (1.0f + expf(-x)); }
-__device__ __forceinline__ float siluf_(float x) { return x / (1.0f + expf(-x)); }
-__device__ __forceinline__ float softplusf_(float x) { return x > 20.0f ? x : log1pf(expf(x)); }
 
 // ------------------------------------------------------------------ token shift
 // out[m][t][c] = x[t][c] + (prev[t][c] - x[t][c]) * mu[m][c], prev = the row of the token
@@ -54,20 +50,22 @@ __global__ void shift_mix_kernel(TX* __restrict__ out, const TX* __restrict__ x,
 // needs of the old tail and then writes, so a step shorter than the tail shifts it in place.
 template <typename TX>
 __global__ void tail_update_kernel(float* __restrict__ state, long long state_stride,
-                                   const TX* __restrict__ x, long long ldx, int C, int R,
+                                   const TX* __restrict__ x, long long ldx,
+                                   const float* __restrict__ bias, int C, int R,
                                    const int* __restrict__ cu, const int* __restrict__ slots) {
   const int s = blockIdx.y;
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   if (c >= C) return;
   const int t0 = cu[s], n = cu[s + 1] - t0;
   float* tail = state + (long long)slots[s] * state_stride;
+  const float b = bias ? bias[c] : 0.f;        // (what the kept rows are: x, or x + bias)
   float keep[kMaxTaps];
 #pragma unroll
   for (int r = 0; r < kMaxTaps; ++r) {
     if (r < R) {
       const int src = n + r;          // index into (old tail ++ new rows) of the row kept at r
       keep[r] = src < R ? tail[(long long)src * C + c]
-                        : ld(x + (long long)(t0 + src - R) * ldx + c);
+                        : ld(x + (long long)(t0 + src - R) * ldx + c) + b;
     }
   }
 #pragma unroll
@@ -77,7 +75,8 @@ __global__ void tail_update_kernel(float* __restrict__ state, long long state_st
 
 // ------------------------------------------- short causal convolution + SiLU (+ unit norm)
 // y[t][c] = act(bias[c] + sum_j taps[c][j] * x[t - (K - 1) + j][c]) (bias optional; act is SiLU,
-// or nothing with activation 0); channels from blend_from on are then mixed with another
+// or nothing with activation 0; with in_bias the inputs are x + in_bias, and so are the tail's
+// rows as tail_update keeps them); channels from blend_from on are then mixed with another
 // tensor's rows of the same tokens, y <- (1 - blend_weight) y + blend_weight * blend[t][c -
 // blend_from] (blend null: no mixing); rows in front of the step come from
 // the tail, rows in front of the sequence are the tail's zeros.  Channels [0, unit_channels)
@@ -86,12 +85,11 @@ __global__ void tail_update_kernel(float* __restrict__ state, long long state_st
 // rest_group for the grid only.  One wave per (token, group), up to 16 channels per lane; a
 // workgroup is four groups of one token.  Both candidates of an input row (the step's, the
 // tail's) are asked for from addresses that exist, and the value is chosen.
-__device__ __forceinline__ float lanes_sum(float v);
-
 template <typename TO>
 __global__ __launch_bounds__(256) void causal_conv_kernel(
     TO* __restrict__ out, const float* __restrict__ x, long long ldx,
-    const float* __restrict__ taps, const float* __restrict__ bias, int C, int K,
+    const float* __restrict__ taps, const float* __restrict__ bias,
+    const float* __restrict__ in_bias, int C, int K,
     const float* __restrict__ state, long long state_stride,
     const int* __restrict__ seq_of_token, const int* __restrict__ cu,
     const int* __restrict__ slots, int unit_channels, int unit_group, int scaled_channels,
@@ -125,12 +123,13 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
       const int off = lane + v * kWave;
       const int c = c0 + (off < width ? off : width - 1);
       float acc = bias ? bias[c] : 0.f;
+      const float shift = in_bias ? in_bias[c] : 0.f;
       for (int j = 0; j < K; ++j) {
         const int back = R - j;              // how many rows before t
         const bool here = back <= rel;
         const float from_step = x[(long long)(t - (here ? back : 0)) * ldx + c];
         const float from_tail = R > 0 ? tail[(long long)(here ? 0 : R - (back - rel)) * C + c] : 0.f;
-        acc += taps[(long long)c * K + j] * (here ? from_step : from_tail);
+        acc += taps[(long long)c * K + j] * (here ? from_step + shift : from_tail);
       }
       if (activation) acc = siluf_(acc);
       if (blend && c >= blend_from)
@@ -154,65 +153,12 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
 }
 
 // ------------------------------------------------------------------ the two scans
-// Sum over the 64 lanes of a wave, every lane gets it: four data-parallel-primitive adds inside
-// rows of 16 lanes (neighbour, pair, the other quad, the other half-row) and the two half
-// swaps; no trip through LDS.  The order of the additions is fixed.
-template <int CTRL>
-__device__ __forceinline__ float dpp_from(float v) {
-  return __int_as_float(__builtin_amdgcn_update_dpp(0, __float_as_int(v), CTRL, 0xF, 0xF, true));
-}
-__device__ __forceinline__ float lanes_sum(float v) {   // (declared above, for the convolution)
-  v += dpp_from<0xB1>(v);    // quad_perm [1, 0, 3, 2]
-  v += dpp_from<0x4E>(v);    // quad_perm [2, 3, 0, 1]
-  v += dpp_from<0x141>(v);   // row_half_mirror
-  v += dpp_from<0x140>(v);   // row_mirror
-  v = xor16_sum(v);
-  return xor32_sum(v);
-}
-
-// Four sums over the wave at once, for values a wave holds per lane for four columns: lanes
-// trade columns with their neighbour and their neighbour's neighbour, so that lane l carries on
-// with column l % 4 alone, and the steps that follow (4 and 8 lanes round the row, the half
-// swaps) keep that class.  Lane l ends with the whole sum of column l % 4: ten adds and moves
-// for four sums where four separate sums take twenty-four.  The order of the additions is fixed.
-__device__ __forceinline__ float lanes_sum4(const float (&p)[4], int lane) {
-  const bool odd = lane & 1, high = lane & 2;
-  float a01 = odd ? p[1] : p[0];
-  a01 += dpp_from<0xB1>(odd ? p[0] : p[1]);
-  float a23 = odd ? p[3] : p[2];
-  a23 += dpp_from<0xB1>(odd ? p[2] : p[3]);
-  float a = high ? a23 : a01;
-  a += dpp_from<0x4E>(high ? a01 : a23);
-  a += dpp_from<0x124>(a);   // row_ror 4
-  a += dpp_from<0x128>(a);   // row_ror 8
-  a = xor16_sum(a);
-  return xor32_sum(a);
-}
-
-// The same for two columns: lane l ends with the whole sum of column l % 2.
-__device__ __forceinline__ float lanes_sum2(const float (&p)[2], int lane) {
-  const bool odd = lane & 1;
-  float a = odd ? p[1] : p[0];
-  a += dpp_from<0xB1>(odd ? p[0] : p[1]);
-  a += dpp_from<0x4E>(a);    // two lanes on: the same column
-  a += dpp_from<0x124>(a);
-  a += dpp_from<0x128>(a);
-  a = xor16_sum(a);
-  return xor32_sum(a);
-}
-template <int NC>
-__device__ __forceinline__ float lanes_sum_cols(const float (&p)[NC], int lane) {
-  if constexpr (NC == 4) return lanes_sum4(p, lane);
-  else return lanes_sum2(p, lane);
-}
-
 // A wave walks kCols value channels of one (sequence, head): lane i holds S[i][j] of each (and
 // i + 64, ... for more than 64 key channels), so what a token brings per key channel is loaded
 // once for all of them and their sums over the wave interleave.  What does not depend on the
 // state (decays, step sizes, the products of a token's own vectors) is made one token ahead,
 // while the token before it waits for its sums.  No load stands under a condition: lanes and
 // columns past the end read a clamped address and their values are zeroed or not stored.
-constexpr int kCols = 4;
 
 // Gated delta rule.  Per token and head, with one decay g and one step size beta per head:
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q.
@@ -421,12 +367,6 @@ __global__ __launch_bounds__(256) void decay_scan_kernel(
 // step sizes; columns and tokens past the end read clamped addresses).  A token's four sums over
 // the wave are formed together (lanes_sum4), so a row comes out as above to rounding, not to
 // the bit.
-template <int KR>
-struct ScanTile {
-  static constexpr int kTokens = KR == 4 ? 16 : 32;
-  static constexpr int kKeys = KR * kWave;
-};
-
 #ifndef RLIS_DELTA_GROUP
 #define RLIS_DELTA_GROUP 2
 #endif
@@ -836,17 +776,6 @@ __global__ __launch_bounds__(256) void head_norm_gate_wide_kernel(
 }  // namespace
 
 // ============================================================================ entry points
-static int scan_compute_units() {
-  static int units = 0;
-  if (units == 0) {
-    int dev = 0;
-    hipDeviceProp_t prop;
-    units = (hipGetDevice(&dev) == hipSuccess && hipGetDeviceProperties(&prop, dev) == hipSuccess)
-                ? prop.multiProcessorCount : 256;
-  }
-  return units;
-}
-
 RLIS_API int rlis_shift_mix(void* out, const void* x, int dtype, const float* mu,
                             const float* state, long long state_stride, const int* seq_of_token,
                             const int* cu, const int* slots, int T, int W, int mixes,
@@ -871,8 +800,8 @@ RLIS_API int rlis_shift_mix(void* out, const void* x, int dtype, const float* mu
 }
 
 RLIS_API int rlis_tail_update(float* state, long long state_stride, const void* x, int dtype,
-                              long long ldx, int C, int R, const int* cu, const int* slots,
-                              int num_seqs, hipStream_t stream) {
+                              long long ldx, const float* bias, int C, int R, const int* cu,
+                              const int* slots, int num_seqs, hipStream_t stream) {
   RLIS_REQUIRE(C > 0 && R >= 0 && R <= 16, "tail_update: bad sizes C=%d rows=%d (at most 16)", C, R);
   RLIS_REQUIRE(state_stride >= (long long)C * R && ldx >= C, "tail_update: strides too short");
   RLIS_REQUIRE(num_seqs <= 65535, "tail_update: %d sequences, at most 65535", num_seqs);
@@ -880,10 +809,10 @@ RLIS_API int rlis_tail_update(float* state, long long state_stride, const void* 
   const dim3 grid(ceil_div(C, 256), num_seqs);
   if (dtype == RLIS_F32)
     tail_update_kernel<float><<<grid, 256, 0, stream>>>(state, state_stride, (const float*)x, ldx,
-                                                        C, R, cu, slots);
+                                                        bias, C, R, cu, slots);
   else if (dtype == RLIS_BF16)
     tail_update_kernel<bf16_t><<<grid, 256, 0, stream>>>(state, state_stride, (const bf16_t*)x,
-                                                         ldx, C, R, cu, slots);
+                                                         ldx, bias, C, R, cu, slots);
   else
     RLIS_REQUIRE(false, "tail_update: unknown dtype %d", dtype);
   RLIS_LAUNCH_CHECK("tail_update");
@@ -891,8 +820,8 @@ RLIS_API int rlis_tail_update(float* state, long long state_stride, const void* 
 }
 
 RLIS_API int rlis_causal_conv(void* out, int out_dtype, const float* x, long long ldx, const float* taps,
-                              const float* bias, int C, int K, const float* state,
-                              long long state_stride,
+                              const float* bias, const float* in_bias, int C, int K,
+                              const float* state, long long state_stride,
                               const int* seq_of_token, const int* cu, const int* slots, int T,
                               int unit_channels, int unit_group, int scaled_channels, float scale,
                               float unit_eps, int rest_group, int activation, const void* blend,
@@ -916,7 +845,7 @@ RLIS_API int rlis_causal_conv(void* out, int out_dtype, const float* x, long lon
   RLIS_REQUIRE(ceil_div(groups, 4) <= 65535, "causal_conv: too many groups");
 #define LAUNCH(TO)                                                                           \
   causal_conv_kernel<TO><<<dim3(T, ceil_div(groups, 4)), 256, 0, stream>>>(                    \
-      (TO*)out, x, ldx, taps, bias, C, K, state, state_stride, seq_of_token, cu, slots,        \
+      (TO*)out, x, ldx, taps, bias, in_bias, C, K, state, state_stride, seq_of_token, cu, slots,        \
       unit_channels, unit_group, scaled_channels, scale, unit_eps,                             \
       rest_group > 0 ? rest_group : 1, groups, activation, (const TO*)blend, ld_blend,         \
       blend_from, blend_weight)

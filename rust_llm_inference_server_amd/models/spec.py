@@ -149,6 +149,11 @@ class Model:
         self.bindings: List[RunBinding] = []
         by_key: Dict[Any, int] = {}
         state_total = 0
+        self.embedding_binding = RunBinding()
+        nbytes = int(self.embedding.state_bytes())
+        if nbytes:
+            self.embedding_binding = RunBinding(state_offset=0, state_bytes=nbytes)
+            state_total = -(-nbytes // 16) * 16
         for i, run in enumerate(self.runs):
             mixer = self.layers[run.layer].mixer
             b = RunBinding()
@@ -183,7 +188,12 @@ class Model:
             raise ValueError(f"sequence of {step.max_context} positions exceeds the model's "
                              f"{rows} learned positions")
         step.carried.clear()
-        stream = ResidualStream(self.embedding.forward(step.ids, step.positions), self.act_dtype)
+        if self.embedding.wants_step:
+            x = self.embedding.forward(step.ids, step.positions, step=step,
+                                       binding=pools.binding(self.embedding_binding))
+        else:
+            x = self.embedding.forward(step.ids, step.positions)
+        stream = ResidualStream(x, self.act_dtype)
         for i, run in enumerate(self.runs):
             self.layers[run.layer].forward(stream, step, pools.binding(self.bindings[i]))
         if step.num_logit_rows == 0:

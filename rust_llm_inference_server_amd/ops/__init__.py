@@ -478,6 +478,122 @@ def swiglu(gu: torch.Tensor) -> torch.Tensor:
     return out
 
 
+def geglu(gu: torch.Tensor) -> torch.Tensor:
+    """``gelu(gu[:, :I]) * gu[:, I:]`` for ``gu`` of shape ``(T, 2 I)`` (tanh form of GELU)."""
+    _check(gu, "gate/up", ndim=2)
+    T, two_i = gu.shape
+    if two_i % 2 or not gu.is_contiguous():
+        raise KernelError("geglu: input must be contiguous with an even number of columns")
+    out = torch.empty((T, two_i // 2), dtype=gu.dtype, device=gu.device)
+    lib.call("rlis_geglu", out.data_ptr(), gu.data_ptr(), _dt(gu), T, two_i // 2, lib.stream_ptr())
+    return out
+
+
+def norm_join(resid: torch.Tensor, y: Optional[torch.Tensor], weight: Optional[torch.Tensor],
+              eps: float, out_dtype: Optional[torch.dtype] = None, round_parts: bool = False
+              ) -> Optional[torch.Tensor]:
+    """``resid += y / sqrt(mean(y^2) + eps) * weight`` row by row in the float32 residual
+    ``(T, W)``; ``y`` is ``(T, W)``, or a stack ``(S, T, W)`` of float32 partial sums that are added in
+    order and with ``round_parts`` rounded to bfloat16 first.  Returns the new residual in
+    ``out_dtype`` (the residual itself for float32, None for None).  ``y`` None: the residual
+    stays as it is."""
+    _check(resid, "residual", torch.float32, 2)
+    if not resid.is_contiguous():
+        raise KernelError("norm_join: residual must be contiguous")
+    T, W = resid.shape
+    if y is None:
+        if out_dtype in (None, torch.float32):
+            return None if out_dtype is None else resid
+        parts, y_args, w_args = 1, (None, 0), (None, 0)
+    else:
+        parts = _delta_parts(resid, y, "norm_join")
+        _check(weight, "norm weight", ndim=1)
+        if weight.numel() != W or not weight.is_contiguous():
+            raise KernelError(f"norm_join: weight has {weight.numel()} entries, rows have {W}")
+        y_args, w_args = (y.data_ptr(), _dt(y)), (weight.data_ptr(), _dt(weight))
+    out = None
+    if out_dtype == torch.bfloat16:
+        out = torch.empty((T, W), dtype=torch.bfloat16, device=resid.device)
+    lib.call("rlis_norm_join", resid.data_ptr(), *y_args, parts, T * W,
+             int(bool(round_parts) and y is not None and y.dim() > 2), *w_args, float(eps),
+             None if out is None else out.data_ptr(), _DT[torch.bfloat16], T, W, lib.stream_ptr())
+    return resid if out_dtype == torch.float32 else out
+
+
+def side_gate_(z: torch.Tensor, table: torch.Tensor, column: int, ids: torch.Tensor
+               ) -> torch.Tensor:
+    """``z (T, n) <- gelu(z) * table[ids][:, column:column + n]`` in place (tanh form, float32
+    arithmetic, one rounding); a table of another dtype than z's is refused."""
+    ldz, ldt = _rows_contig(z, "side_gate z"), _rows_contig(table, "side_gate table")
+    T, n = z.shape
+    if table.dtype != z.dtype or not 0 <= column <= table.shape[1] - n:
+        raise KernelError(f"side_gate: columns {column} to {column + n} of a {table.dtype} table of "
+                          f"{table.shape[1]} for {z.dtype} rows")
+    lib.call("rlis_side_gate", z.data_ptr(), _dt(z), ldz,
+             table.data_ptr() + column * table.element_size(), ldt, _i32(ids, "ids", T), T, n,
+             lib.stream_ptr())
+    return z
+
+
+def embed_pairs(ids: torch.Tensor, table: torch.Tensor, scale: float, pairs: torch.Tensor,
+                mul_prev: int, mul_cur: int, last: torch.Tensor, seq_of_token: torch.Tensor,
+                cu: torch.Tensor, slots: torch.Tensor) -> torch.Tensor:
+    """``table[ids] * scale + pairs[row]`` as the float32 stream ``(T, W)`` with ``row = (previous *
+    mul_prev + id * mul_cur) mod n`` for ``pairs (n + 1, W)``, and row n for a sequence's first
+    token.  ``last (slots, >= 1)`` int32 (rows a whole state slot apart) holds each request's last
+    token plus one (0: none yet) and is left as after the step."""
+    _check(table, "embed table", ndim=2)
+    _check(pairs, "pair table", table.dtype, 2)
+    T, (V, W) = ids.numel(), table.shape
+    if not table.is_contiguous() or not pairs.is_contiguous() or pairs.shape[1] != W \
+            or pairs.shape[0] < 2:
+        raise KernelError("embed_pairs: both tables must be contiguous rows of one width")
+    _check(last, "last tokens", torch.int32, 2)
+    out = torch.empty((T, W), dtype=torch.float32, device=table.device)
+    S = cu.numel() - 1
+    lib.call("rlis_embed_pairs", out.data_ptr(), table.data_ptr(), pairs.data_ptr(), _dt(table),
+             _i32(ids, "ids", T), T, W, pairs.shape[0] - 1, float(scale), int(mul_prev),
+             int(mul_cur), last.data_ptr(), last.stride(0), _i32(seq_of_token, "seq_of_token", T),
+             _i32(cu, "cu", S + 1), _i32(slots, "slots", S), lib.stream_ptr())
+    return out
+
+
+def row_prepare(p: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int, real_dim: int,
+                bias: Optional[torch.Tensor], q_weight: torch.Tensor, k_weight: torch.Tensor,
+                eps: float, cos: Optional[torch.Tensor], sin: Optional[torch.Tensor],
+                positions: torch.Tensor, interleaved: bool = False) -> torch.Tensor:
+    """Rows ``[q | k | ...]`` of a projection (heads ``head_dim`` wide, their first ``real_dim``
+    numbers the model's and the rest zeros) as rows ``[q | k | v]`` for the attention kernels:
+    ``v = k + bias``; q and k biased, each divided by the root mean square of the token's whole
+    row of them (eps inside the root), times a float32 weight per column, and rotated by the
+    token's position (the first ``2 * cos.shape[1]`` dims of a head, pairs of neighbours with
+    ``interleaved``, halves without).  Float32 arithmetic, one rounding."""
+    ldp = _rows_contig(p, "row_prepare rows")
+    T, nh, nkv, D = p.shape[0], int(num_heads), int(num_kv_heads), int(head_dim)
+    if p.shape[1] < (nh + nkv) * D:
+        raise KernelError(f"row_prepare: rows of {p.shape[1]} hold no {nh + nkv} heads of {D}")
+    for t, n, what in ((bias, (nh + nkv) * D, "bias"), (q_weight, nh * D, "query weight"),
+                       (k_weight, nkv * D, "key weight")):
+        if t is not None:
+            _check(t, f"row_prepare {what}", torch.float32, 1)
+            if t.numel() != n or not t.is_contiguous():
+                raise KernelError(f"row_prepare: the {what} has {t.numel()} entries, expected {n}")
+    cos_ptr = sin_ptr = None
+    rot = 0
+    if cos is not None:
+        for t in (cos, sin):
+            _check(t, "row_prepare angles", torch.float32, 2)
+        if cos.shape != sin.shape or not (cos.is_contiguous() and sin.is_contiguous()):
+            raise KernelError("row_prepare: cos and sin must match and be contiguous")
+        cos_ptr, sin_ptr, rot = cos.data_ptr(), sin.data_ptr(), 2 * cos.shape[1]
+    out = torch.empty((T, (nh + 2 * nkv) * D), dtype=p.dtype, device=p.device)
+    lib.call("rlis_row_prepare", out.data_ptr(), p.data_ptr(), _dt(p), ldp, T, nh, nkv, D,
+             int(real_dim), None if bias is None else bias.data_ptr(), q_weight.data_ptr(),
+             k_weight.data_ptr(), float(eps), cos_ptr, sin_ptr, rot,
+             _i32(positions, "positions", T), int(bool(interleaved)), lib.stream_ptr())
+    return out
+
+
 def clamped_glu(gu: torch.Tensor, limit: float, alpha: float) -> torch.Tensor:
     """For ``gu = [gate | up]`` of shape ``(T, 2 I)``: ``g * sigmoid(alpha * g) * (u + 1)`` with
     ``g = min(gate, limit)`` and ``u = clamp(up, -limit, limit)``."""
@@ -899,6 +1015,13 @@ def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor) -> torch.Tensor:
     return y
 
 
+def linear_geglu(x: torch.Tensor, w_gate_up: torch.Tensor) -> torch.Tensor:
+    """``gelu(x @ Wg.T) * (x @ Wu.T)`` (tanh form) for ``w_gate_up = [Wg; Wu]`` of ``(2 I, K)``."""
+    if w_gate_up.shape[0] % 2:
+        raise KernelError("linear_geglu: the fused weight needs an even number of rows")
+    return geglu(linear(x, w_gate_up, x.dtype))
+
+
 # ------------------------------------------------------------ rotation + cache write
 def rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
                   cos: Optional[torch.Tensor], sin: Optional[torch.Tensor],
@@ -984,15 +1107,17 @@ PLAIN_EXTRAS = False
 
 def attention_planner(num_heads: int, num_kv_heads: int, head_dim: int,
                       dtype: torch.dtype, biased: bool = False,
-                      shaped: bool = False, plain: bool = False) -> AttentionPlanner:
+                      shaped: bool = False, plain: bool = False,
+                      span: int = 0) -> AttentionPlanner:
     """The planner a mixer that calls ``paged_attention`` / ``rope_attention`` names as its
     ``step_planner()``; ``biased``: it will pass ``bias_slopes`` (the matrix-core kernels take
     them too, so the plan is the same); ``shaped``: it will pass ``head_scales`` or a
-    ``softcap``."""
+    ``softcap``; ``span``: the ``chunk`` it will pass (0: none)."""
     return AttentionPlanner(num_heads, num_kv_heads, head_dim,
                             matrix=dtype == torch.bfloat16 and not (plain and PLAIN_EXTRAS)
                             and (not shaped or SHAPED_SCORES_MATRIX),
-                            singles_apart=SPLIT_MIXED_ATTENTION and DECODE_ATTENTION != "vector")
+                            singles_apart=SPLIT_MIXED_ATTENTION and DECODE_ATTENTION != "vector",
+                            span=span)
 
 
 def _attention_kernel(qkv: torch.Tensor, nh: int, nkv: int, d: int, page_size: int, step,
@@ -1036,9 +1161,9 @@ def rope_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
                    counters: Optional[torch.Tensor] = None,
                    head_scales: Optional[torch.Tensor] = None,
                    softcap: float = 0.0, sinks: Optional[torch.Tensor] = None,
-                   keep_first: int = 0) -> torch.Tensor:
-    """``rope_kv_write`` followed by ``paged_attention`` (``head_scales``, ``softcap``, ``sinks``
-    and ``keep_first`` as there).  ``qkv`` may hold the queries alone (``(T, nh * d)``) when
+                   keep_first: int = 0, chunk: Optional[int] = None) -> torch.Tensor:
+    """``rope_kv_write`` followed by ``paged_attention`` (``head_scales``, ``softcap``, ``sinks``,
+    ``keep_first`` and ``chunk`` as there).  ``qkv`` may hold the queries alone (``(T, nh * d)``) when
     nothing is written to the cache.  A decode batch that takes the
     matrix-core decode kernel does both in that kernel when the whole head is rotated
     (rotate-half) and is 64, 128 or 256 wide (or nothing is rotated); ``qkv`` is then left
@@ -1050,7 +1175,8 @@ def rope_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
     nh, nkv, d = num_heads, num_kv_heads, head_dim
     _rows_contig(qkv, "qkv")
     shaped = head_scales is not None or softcap > 0
-    more = dict(head_scales=head_scales, softcap=softcap, sinks=sinks, keep_first=keep_first)
+    more = dict(head_scales=head_scales, softcap=softcap, sinks=sinks, keep_first=keep_first,
+                chunk=chunk)
     kind, mfma = _attention_kernel(qkv, nh, nkv, d, page_size, step, None, bias_slopes is not None,
                                    shaped, PLAIN_EXTRAS and (sinks is not None
                                                              or bool(keep_first and window)))
@@ -1101,7 +1227,7 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
                     counters: Optional[torch.Tensor] = None,
                     head_scales: Optional[torch.Tensor] = None,
                     softcap: float = 0.0, sinks: Optional[torch.Tensor] = None,
-                    keep_first: int = 0) -> torch.Tensor:
+                    keep_first: int = 0, chunk: Optional[int] = None) -> torch.Tensor:
     """Attention of the step's new tokens over the paged cache -> ``(T, nh * d)``.
 
     ``qkv`` holds the rotated queries in its first ``nh * d`` columns; K and V of the new
@@ -1121,7 +1247,8 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
     ``sinks`` (float32, one per query head): the softmax's denominator also holds ``e^sink`` of
     the head, once, unscaled, with no key and no value behind it.  ``keep_first`` n (with a
     window): the first n keys of a sequence stay visible to every later query, at their own
-    positions, beside the window's keys.
+    positions, beside the window's keys.  ``chunk`` c (without a window): a query at position p
+    sees the keys of its own chunk alone, those up to p with ``floor(key / c) = floor(p / c)``.
     ``force`` names one of 'generic', 'decode', 'prefill' for tests.  ``rope`` (from
     ``rope_attention`` only): ``(cos, sin, positions, slots)`` for the matrix-core decode kernel
     to rotate and store the step's tokens itself; with portions of prompts in the batch
@@ -1152,6 +1279,9 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
     if T != step.num_tokens:
         raise KernelError(f"attention: qkv has {T} rows, the step {step.num_tokens} tokens")
     win = int(window) if window else 0
+    span = int(chunk) if chunk else 0
+    if span < 0 or (span and (win or keep_first)):
+        raise KernelError("attention: a window or chunks of positions, not both")
     out = torch.empty((T, nh * d), dtype=qkv.dtype, device=qkv.device)
     stream = lib.stream_ptr()
     slopes_ptr = None
@@ -1190,14 +1320,14 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
                  k_pages.data_ptr(), v_pages.data_ptr(), block_tables.data_ptr(), max_pages,
                  _i32(step.seq_of_token, "seq_of_token", T), _i32(step.positions, "positions", T),
                  T, nh, nkv, d, page_size, float(scale), win, slopes_ptr, scales_ptr, softcap,
-                 sinks_ptr, kept, stream)
+                 sinks_ptr, kept, span, stream)
         return out
     if kind not in ("decode", "prefill"):
         raise KernelError(f"attention: unknown kernel '{kind}'")
     if plan is None or force == "prefill":
         planner = AttentionPlanner(nh, nkv, d, matrix=qkv.dtype == torch.bfloat16,
                                    singles_apart=force is None and SPLIT_MIXED_ATTENTION
-                                   and DECODE_ATTENTION != "vector")
+                                   and DECODE_ATTENTION != "vector", span=span)
         plan = _plan_now(step, planner, qkv.device)
 
     def decode(S: int, depth: int, matrix: bool) -> None:
@@ -1238,14 +1368,14 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
                      nh, nkv, d, page_size, win, float(scale), depth, ap.DECODE_PART_KEYS,
                      ap.DECODE_MAX_PARTS, arrivals_p, arrival_slots, groups, cap, cos_p, sin_p,
                      rot, pos_p, slots_p, nh * d, (nh + nkv) * d, slopes_ptr, scales_ptr, softcap,
-                     sinks_ptr, kept, stream)
+                     sinks_ptr, kept, span, stream)
         else:
             lib.call("rlis_attn_decode", qkv.data_ptr(), _dt(qkv), q_stride, out.data_ptr(),
                      nh * d, ml_ptr, acc_ptr, k_pages.data_ptr(), v_pages.data_ptr(),
                      block_tables.data_ptr(), max_pages, _i32(step.ctx_lens, "ctx_lens", S), None,
                      S, nh, nkv, d, page_size, float(scale), win, depth, ap.DECODE_PART_KEYS,
                      ap.DECODE_MAX_PARTS, slopes_ptr, scales_ptr, softcap, sinks_ptr, kept,
-                     stream)
+                     span, stream)
 
     if kind == "decode":
         if not step.all_decode:
@@ -1295,7 +1425,7 @@ def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_d
                  _i32(step.start_pos, "start_pos", step.num_seqs),
                  _i32(plan[name], name, 4 * n), n, nh, nkv, d, page_size, win, float(scale), tile,
                  max_runs, row0, ml_ptr, acc_ptr, cos_p, sin_p, rot, slopes_ptr, scales_ptr,
-                 softcap, sinks_ptr, kept, stream)
+                 softcap, sinks_ptr, kept, span, stream)
     if not launched and T > row0:
         raise KernelError("attention: the plan holds no tiles for the step's portions")
     if launched and max_runs > 1:
@@ -1335,8 +1465,9 @@ def sample_rows(logits: torch.Tensor, keys: torch.Tensor, inv_temps: torch.Tenso
     return out
 
 
-from .recurrent import (causal_conv, decay_attention, decay_scan, delta_scan,  # noqa: E402,F401
-                        head_norm_gate, selective_scan, shift_mix, tail_update)
+from .recurrent import (causal_conv, channel_delta_scan, decay_attention, decay_scan,  # noqa: E402,F401
+                        delta_scan, head_norm_gate, rglru_scan, selective_scan, shift_mix,
+                        tail_update)
 from .latent import (head_linear, latent_attention, latent_mfma_ok, latent_write,  # noqa: E402,F401
                      sigmoid_gate_)
 from .routed import routed_units, route, router_logits  # noqa: E402,F401

@@ -97,10 +97,13 @@ class AttentionPlanner(StepPlanner):
     ``matrix``: the batch can take the matrix-core kernels (bfloat16, head size in steps of 16
     up to 256); without it only the depth of the decode grid is planned.  ``singles_apart``:
     sequences that bring one token beside portions of prompts take the decode kernel (they
-    lead the step); otherwise they get tiles like everyone else."""
+    lead the step); otherwise they get tiles like everyone else.  ``span``: the most keys one
+    query sees (chunked attention), 0: all earlier ones; work that cannot be is not cut into
+    pieces."""
 
     def __init__(self, num_heads: int, num_kv_heads: int, head_dim: int, matrix: bool = True,
-                 singles_apart: bool = True):
+                 singles_apart: bool = True, span: int = 0):
+        self.span = int(span)
         self.nh, self.nkv, self.d = int(num_heads), int(num_kv_heads), int(head_dim)
         self.matrix = bool(matrix) and self.d % 16 == 0 and self.d <= 256
         g = self.nh // max(1, self.nkv)
@@ -110,7 +113,12 @@ class AttentionPlanner(StepPlanner):
                               and g * (self.d + 2) * 32 <= 65536)
 
     def key(self) -> Any:
-        return ("attention", self.nh, self.nkv, self.d, self.matrix, self.singles_apart)
+        return ("attention", self.nh, self.nkv, self.d, self.matrix, self.singles_apart, self.span)
+
+    def _reach(self, context: int) -> int:
+        """Keys that a decoded token of ``context`` positions may walk (the matrix-core kernel
+        starts at a multiple of 32)."""
+        return min(context, self.span + 31) if self.span else context
 
     @staticmethod
     def pages_fit(page_size: int) -> bool:
@@ -122,6 +130,7 @@ class AttentionPlanner(StepPlanner):
         """64 or 128: the tile form of a sequence with ``cached`` positions and ``new`` tokens."""
         if self.d > 128 or PREFILL_WIDE_MIN_GROUPS >= (1 << 30):
             return PREFILL_TILE
+        cached = min(cached, self.span) if self.span else cached
         groups = -(-new // WIDE_TILE) * self.nh
         enough = PREFILL_WIDE_MIN_GROUPS if self.d > 64 else PREFILL_WIDE_MIN_GROUPS * 5 // 3
         if groups >= enough or cached + new >= 4096 or cached >= 2048:
@@ -130,6 +139,7 @@ class AttentionPlanner(StepPlanner):
 
     def key_runs(self, cached: int, new: int, tile: int) -> int:
         """Runs the keys of this sequence's tiles are cut into (1: none)."""
+        cached = min(cached, self.span) if self.span else cached
         groups = -(-new // tile) * self.nh
         if PREFILL_SPLIT_UNITS <= 0 or groups > PREFILL_SPLIT_UNITS:
             return 1
@@ -156,6 +166,8 @@ class AttentionPlanner(StepPlanner):
             runs[s] = r
             qb = np.arange(0, n, tile, dtype=np.int64)
             keys = c + np.minimum(n, qb + tile)                # keys a tile walks
+            if self.span:
+                keys = np.minimum(keys, (c + qb) % self.span + tile)
             u = np.empty((len(qb), r, 5), dtype=np.int64)
             u[:, :, 0] = s
             u[:, :, 1] = qb[:, None]
@@ -177,11 +189,13 @@ class AttentionPlanner(StepPlanner):
         values["tile_row0"] = int(new[:singles].sum())         # rows before the tiles' rows
         values["num_decode"] = singles
         ctx = start + new
-        values["decode_depth"] = decode_depth(int(ctx[:singles].max()) if singles else 1)
+        values["decode_depth"] = decode_depth(self._reach(int(ctx[:singles].max()))
+                                              if singles else 1)
         return HostPlan(arrays, values)
 
     def plan_captured(self, num_seqs: int, max_context: int, page_size: int) -> HostPlan:
-        return HostPlan({}, {"decode_depth": decode_depth(max_context), "num_decode": num_seqs,
+        return HostPlan({}, {"decode_depth": decode_depth(self._reach(max_context)),
+                             "num_decode": num_seqs,
                              "max_runs": 1, "tile_row0": num_seqs, "num_units64": 0,
                              "num_units128": 0})
 

@@ -29,12 +29,19 @@ _SIGNATURES = {
     "rlis_add_residual": [P, P, I, L, I, I, F, P],
     "rlis_add_rmsnorm": [P, P, I, P, I, P, I, P, I, I, F, I, I, L, I, F, P],
     "rlis_swiglu": [P, P, I, I, I, P],
+    "rlis_geglu": [P, P, I, I, I, P],
+    "rlis_norm_join": [P, P, I, I, L, I, P, I, F, P, I, I, I, P],
+    "rlis_side_gate": [P, I, L, P, L, P, I, I, P],
+    "rlis_embed_pairs": [P, P, P, I, P, I, I, I, F, L, L, P, L, P, P, P, P],
+    "rlis_row_prepare": [P, P, I, L, I, I, I, I, I, P, P, P, F, P, P, I, P, I, P],
+    "rlis_channel_delta_scan": [P, L, P, P, P, L, P, L, P, L, P, P, P, L, P, P, I, I, I, I, I, I, P],
+    "rlis_rglru_scan": [P, I, P, L, P, L, P, P, P, P, L, P, P, L, P, P, I, I, I, I, I, P, P],
     "rlis_clamped_glu": [P, P, I, I, I, F, F, P],
     "rlis_weighted_sum": [P, P, I, F, I, P, I, F, I, L, I, P],
     "rlis_soft_cap": [P, I, L, F, P],
     "rlis_shift_mix": [P, P, I, P, P, L, P, P, P, I, I, I, P],
-    "rlis_tail_update": [P, L, P, I, L, I, I, P, P, I, P],
-    "rlis_causal_conv": [P, I, P, L, P, P, I, I, P, L, P, P, P, I, I, I, I, F, F, I, I, P, L, I, F, P],
+    "rlis_tail_update": [P, L, P, I, L, P, I, I, P, P, I, P],
+    "rlis_causal_conv": [P, I, P, L, P, P, P, I, I, P, L, P, P, P, I, I, I, I, F, F, I, I, P, L, I, F, P],
     "rlis_selective_scan": [P, I, L, P, L, P, L, P, P, P, L, P, L, P, P, P, L, P, P, I, I, I, I, I, I,
                             P, P, P],
     "rlis_add_layernorm": [P, P, I, P, P, I, P, I, P, I, I, F, I, I, L, I, F, P],
@@ -63,13 +70,13 @@ _SIGNATURES = {
     "rlis_gemm_bf16_stream_join": [P, P, I, I, I, L, L, P, P, P, I, I, P, P, I, P],
     "rlis_gemm_bf16_stream_scaled": [P, P, P, I, I, I, I, L, L, L, I, P, I, I, F, P],
     "rlis_norm_linear_bf16": [P, P, I, I, L, I, P, I, F, P, P, P, P, I, I, I, I, L, L, I, P],
-    "rlis_attn_generic": [P, I, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, P, P, F, P, I, P],
+    "rlis_attn_generic": [P, I, L, P, L, P, P, P, I, P, P, I, I, I, I, I, F, I, P, P, F, P, I, I, P],
     "rlis_attn_decode": [P, I, L, P, L, P, P, P, P, P, I, P, P, I, I, I, I, I, F, I, I, I, I, P, P, F,
-                         P, I, P],
+                         P, I, I, P],
     "rlis_attn_decode_mfma": [P, L, P, L, P, P, P, P, P, I, P, I, I, I, I, I, I, F, I, I, I, P, I, I, I,
-                              P, P, I, P, P, L, L, P, P, F, P, I, P],
+                              P, P, I, P, P, L, L, P, P, F, P, I, I, P],
     "rlis_attn_prefill_mfma": [P, L, P, L, P, P, P, I, P, P, P, I, I, I, I, I, I, F, I, I, I, P, P,
-                               P, P, I, P, P, F, P, I, P],
+                               P, P, I, P, P, F, P, I, I, P],
     "rlis_attn_reduce_rows": [P, L, P, P, P, P, I, I, I, I, I, P, P],
     "rlis_sample_rows": [P, L, I, I, P, P, P, I, P, P, P],
     "rlis_fill_normal_device": [P, I, L, ctypes.c_ulonglong, ctypes.c_ulonglong, ctypes.c_double,

@@ -93,15 +93,17 @@ def shift_mix(x: torch.Tensor, mu: torch.Tensor, state: torch.Tensor, seq_of_tok
 
 
 def tail_update(state: torch.Tensor, x: torch.Tensor, channels: int, rows: int, cu: torch.Tensor,
-                slots: torch.Tensor, num_seqs: int) -> None:
+                slots: torch.Tensor, num_seqs: int, bias: Optional[torch.Tensor] = None) -> None:
     """Every sequence's tail in ``state`` (``rows`` rows of ``channels`` floats, oldest first)
-    becomes the last ``rows`` of (its old tail, then the step's rows of ``x[:, :channels]``)."""
+    becomes the last ``rows`` of (its old tail, then the step's rows of ``x[:, :channels]``, plus
+    ``bias`` (float32, one per channel) when given)."""
     ldx = _rows(x, "tail_update x")
     if x.shape[1] < channels:
         raise KernelError(f"tail_update: x has {x.shape[1]} columns, {channels} needed")
     stride = _state(state, channels * rows, "tail_update")
-    lib.call("rlis_tail_update", state.data_ptr(), stride, x.data_ptr(), _dt(x), ldx, channels,
-             rows, _meta(cu, num_seqs + 1, "cu"), _meta(slots, num_seqs, "slots"), num_seqs,
+    lib.call("rlis_tail_update", state.data_ptr(), stride, x.data_ptr(), _dt(x), ldx,
+             None if bias is None else _vec(bias, channels, "tail_update bias"), channels, rows,
+             _meta(cu, num_seqs + 1, "cu"), _meta(slots, num_seqs, "slots"), num_seqs,
              lib.stream_ptr())
 
 
@@ -112,10 +114,13 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor,
                 bias: Optional[torch.Tensor] = None,
                 out_dtype: torch.dtype = torch.float32, activation: bool = True,
                 blend: Optional[torch.Tensor] = None, blend_from: int = 0,
-                blend_weight: float = 0.0) -> torch.Tensor:
+                blend_weight: float = 0.0,
+                in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
     """``silu`` of the causal convolution over time of the first ``C`` columns of ``x`` (float32)
     with ``taps (C, K)`` (the last column multiplies the current row; the ``K - 1`` rows in
-    front of the step come from ``state``), plus ``bias (C)`` under the ``silu`` when given;
+    front of the step come from ``state``), plus ``bias (C)`` under the ``silu`` when given
+    (``in_bias (C)``: the inputs are ``x + in_bias``, as are the rows that ``tail_update`` keeps
+    with that bias);
     without ``activation`` the convolution as it is.  With ``blend`` (rows of the same tokens in
     ``out_dtype``, ``C - blend_from`` columns) the channels from ``blend_from`` on become
     ``(1 - blend_weight) * y + blend_weight * blend``.  Channels below ``unit_channels`` are then made
@@ -137,7 +142,8 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor,
                               f"channels {blend_from} to {C} of {T} tokens")
         blend_ptr = blend.data_ptr()
     lib.call("rlis_causal_conv", out.data_ptr(), _DT[out_dtype], x.data_ptr(), ldx,
-             taps.data_ptr(), None if bias is None else _vec(bias, C, "causal_conv bias"), C, K,
+             taps.data_ptr(), None if bias is None else _vec(bias, C, "causal_conv bias"),
+             None if in_bias is None else _vec(in_bias, C, "causal_conv input bias"), C, K,
              state.data_ptr(), stride, _meta(seq_of_token, T, "seq_of_token"),
              _meta(cu, num_seqs + 1, "cu"), _meta(slots, num_seqs, "slots"), T,
              int(unit_channels), int(unit_group), int(scaled_channels), float(scale),
@@ -231,6 +237,77 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, he
     lib.call("rlis_head_norm_gate", out.data_ptr(), _DT[out_dtype], o.data_ptr(),
              weight.data_ptr(), wstride, gate.data_ptr(), _dt(gate), ldg, T, heads, dv, float(eps),
              int(bool(sigmoid_gate)), lib.stream_ptr())
+    return out
+
+
+def channel_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b_raw: torch.Tensor,
+                       z: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor,
+                       state: torch.Tensor, cu: torch.Tensor, slots: torch.Tensor, num_seqs: int,
+                       heads: int, kv_heads: int, dk: int, dv: int, tiled=None) -> torch.Tensor:
+    """``delta_scan`` with one decay per head and key channel: per token and head
+    ``S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q`` with
+    ``g[i] = exp(-exp(a_log[head]) * softplus(z[head * dk + i] + dt_bias[head * dk + i]))`` and
+    ``beta = sigmoid(b_raw)``.  ``z (T, heads * dk)``, ``b_raw (T, heads)`` float32 with rows of
+    their own strides; everything else as for ``delta_scan``."""
+    ld = _rows(q, "channel_delta_scan q", torch.float32)
+    if _rows(k, "channel_delta_scan k", torch.float32) != ld \
+            or _rows(v, "channel_delta_scan v", torch.float32) != ld:
+        raise KernelError("channel_delta_scan: q, k and v must share a row stride")
+    ldb = _rows(b_raw, "channel_delta_scan b", torch.float32)
+    ldz = _rows(z, "channel_delta_scan z", torch.float32)
+    T = q.shape[0]
+    if q.shape[1] != kv_heads * dk or k.shape != q.shape or v.shape != (T, heads * dv) \
+            or b_raw.shape != (T, heads) or z.shape != (T, heads * dk):
+        raise KernelError("channel_delta_scan: operand shapes do not match the head counts and sizes")
+    stride = _state(state, heads * dv * dk, "channel_delta_scan")
+    out = torch.empty((T, heads * dv), dtype=torch.float32, device=q.device)
+    lib.call("rlis_channel_delta_scan", out.data_ptr(), heads * dv, q.data_ptr(), k.data_ptr(),
+             v.data_ptr(), ld, b_raw.data_ptr(), ldb, z.data_ptr(), ldz,
+             _vec(a_log, heads, "channel_delta_scan A_log"),
+             _vec(dt_bias, heads * dk, "channel_delta_scan dt_bias"),
+             state.data_ptr(), stride, _meta(cu, num_seqs + 1, "cu"),
+             _meta(slots, num_seqs, "slots"), num_seqs, heads, kv_heads, dk, dv,
+             _scan_form(tiled, T, num_seqs), lib.stream_ptr())
+    return out
+
+
+# A step in which some sequence brings at least RGLRU_CHUNKED_MIN_LONGEST tokens takes the chunked
+# form of the gated linear recurrence: chunks of RGLRU_CHUNK_LEN tokens side by side from zero, the
+# chunks' states joined in order, every chunk again from its true start (the recurrence is linear
+# in the state).  It agrees with the walk token by token to rounding.
+RGLRU_CHUNK_LEN = 32
+RGLRU_CHUNKED_MIN_LONGEST = 96
+
+
+def rglru_scan(u: torch.Tensor, gates: torch.Tensor, r_bias: torch.Tensor, i_bias: torch.Tensor,
+               rate: torch.Tensor, y: torch.Tensor, y_bias: torch.Tensor, state: torch.Tensor,
+               cu: torch.Tensor, slots: torch.Tensor, num_seqs: int, blocks: int,
+               longest: Optional[int] = None) -> torch.Tensor:
+    """A gated linear recurrence per channel over every sequence's tokens of the step: ``r, i =
+    sigmoid(gates + biases)``, ``log a = rate r``, ``S <- a S + sqrt(1 - a^2) i u``, result
+    ``S * gelu(y + y_bias)`` (tanh form).  ``u (T, C)`` is in the activation dtype and so is the
+    result; ``gates (T, 2 C)`` float32 holds per block of ``n = C / blocks`` channels n numbers
+    for r and then n for i; ``y (T, C)`` float32 with a row stride; biases and ``rate`` float32
+    ``(C)``.  ``state (slots, C)`` is left as after each sequence's last token.  ``longest``: the
+    most tokens a sequence brings, where known (None: ``T``)."""
+    T, C = u.shape
+    ldu, ldy = _rows(u, "rglru_scan u"), _rows(y, "rglru_scan y", torch.float32)
+    ldg = _rows(gates, "rglru_scan gates", torch.float32)
+    if C % blocks or gates.shape != (T, 2 * C) or y.shape != (T, C):
+        raise KernelError("rglru_scan: operand shapes do not match the channels and blocks")
+    stride = _state(state, C, "rglru_scan")
+    out = torch.empty((T, C), dtype=u.dtype, device=u.device)
+    max_chunks, ws = 0, None
+    if (T if longest is None else longest) >= RGLRU_CHUNKED_MIN_LONGEST:
+        max_chunks = T // RGLRU_CHUNK_LEN + num_seqs            # an upper bound, known on the host
+        ws = torch.empty((2, max_chunks, C), dtype=torch.float32, device=u.device)
+    lib.call("rlis_rglru_scan", out.data_ptr(), _dt(u), u.data_ptr(), ldu, gates.data_ptr(), ldg,
+             _vec(r_bias, C, "rglru_scan r bias"), _vec(i_bias, C, "rglru_scan i bias"),
+             _vec(rate, C, "rglru_scan rate"), y.data_ptr(), ldy,
+             _vec(y_bias, C, "rglru_scan y bias"), state.data_ptr(), stride,
+             _meta(cu, num_seqs + 1, "cu"), _meta(slots, num_seqs, "slots"), num_seqs, C,
+             C // blocks, RGLRU_CHUNK_LEN, max_chunks, None if ws is None else ws.data_ptr(),
+             lib.stream_ptr())
     return out
 
 

@@ -1,8 +1,8 @@
 """The parts a model is put together from.  Importing the package registers the built-in
 kinds: mixers ``attention``, ``latent_attention``, ``time_mix``, ``gated_delta``,
-``selective_scan`` and ``parallel``; feed-forwards ``swiglu``, ``clamped_glu`` and
-``routed_swiglu``; norms ``rmsnorm`` and ``layernorm``; position ``rope`` and ``none``; blocks
-``prenorm`` and ``parallel``; embedding ``token``; head ``linear``."""
+``selective_scan``, ``decay_attention``, ``channel_delta``, ``rglru`` and ``parallel``; feed-forwards ``swiglu``, ``mlp``, ``gated_mlp``,
+``clamped_glu``, ``token_side``, ``routed_swiglu`` and ``routed_mlp``; norms ``rmsnorm`` and ``layernorm``; position ``rope`` and ``none``; blocks
+``prenorm``, ``postnorm``, ``hyper`` and ``parallel``; embedding ``token``; head ``linear``."""
 from . import attention, block, embedding, latent, mlp, norm, recurrent, rope  # noqa: F401  (registration)
 from .base import (Block, BuildContext, CacheBinding, CacheRequest, Embedding, FeedForward,
                    Head, Mixer, Norm, NormedInput, Part, PartSpec, PositionEncoding,

@@ -53,6 +53,16 @@ class PagedAttention(Mixer):
     * ``keep_first`` n (with a ``window``): the first n keys of a sequence stay visible to every
       later query beside the window's keys, at their own positions; the cache keeps their pages
       while it gives back those that the window has passed.
+    * ``chunk`` c (no ``window`` then): a query at position p sees the keys of its own chunk of c
+      positions only, j <= p with ``floor(j / c) = floor(p / c)``, chunks counted from position 0.
+      The cache keeps the last c positions, which hold the query's chunk whatever its place.
+    * ``keys_as_values``: the layer has no value projection; the values are the keys as the
+      projection (with its bias) gives them, in front of norm and rotation.
+    * ``qk_norm`` with ``"whole": True``: the norm runs over a token's whole row of queries (and
+      of keys) at once, in front of the cut into heads; the weights have the row's size.
+    * ``channel_gate``: the name of a projection ``(num_heads * value_dim, hidden_size)`` of the
+      mixer's input; its sigmoid multiplies the concatenated heads element by element, in front
+      of the output projection.
     * ``gate``: the name of a projection ``(num_heads, hidden_size)`` of the mixer's input: head
       h of the result is multiplied by the sigmoid of output h, in front of the output
       projection.
@@ -90,17 +100,24 @@ class PagedAttention(Mixer):
         dv = params.get("value_dim") or d
         n = cls._names(params, prefix)
         own_kv = not params.get("shared_kv")
+        own_v = own_kv and not params.get("keys_as_values")
         out = [TensorSpec(n["q"], (nh * d, H))]
         if own_kv:
-            out += [TensorSpec(n["k"], (nkv * d, H)), TensorSpec(n["v"], (nkv * dv, H))]
+            out.append(TensorSpec(n["k"], (nkv * d, H)))
+        if own_v:
+            out.append(TensorSpec(n["v"], (nkv * dv, H)))
         out.append(TensorSpec(n["o"], (H, nh * dv)))
         if params.get("bias"):
             out += [TensorSpec(n[c] + params["bias"], (rows,), std=0.1) for c, rows in
-                    (("q", nh * d), ("k", nkv * d), ("v", nkv * dv)) if c == "q" or own_kv]
+                    (("q", nh * d), ("k", nkv * d), ("v", nkv * dv))
+                    if c == "q" or (own_v if c == "v" else own_kv)]
         norm = params.get("qk_norm")
         if norm:
-            out += [TensorSpec(join(prefix, norm[c]), (d,), init="ones_normal", std=0.1)
+            size = {"q": nh * d, "k": nkv * d} if norm.get("whole") else {"q": d, "k": d}
+            out += [TensorSpec(join(prefix, norm[c]), (size[c],), init="ones_normal", std=0.1)
                     for c in "qk" if c == "q" or own_kv]
+        if params.get("channel_gate"):
+            out.append(TensorSpec(join(prefix, params["channel_gate"]), (nh * dv, H)))
         if params.get("sinks"):
             out.append(TensorSpec(join(prefix, params["sinks"]), (nh,), std=1.0))
         if params.get("gate"):
@@ -149,12 +166,33 @@ class PagedAttention(Mixer):
         names = self._names(params, prefix)
         self.shared_kv = bool(params.get("shared_kv"))
         self.qk_dim = qk_dim
+        self.chunk: Optional[int] = params.get("chunk")
+        self.keys_as_values = bool(params.get("keys_as_values"))
+        norm = params.get("qk_norm") or {}
+        self.whole_norm = bool(norm.get("whole"))
+        # the layer's rows are laid out (and rotated) by one kernel in front of the attention
+        self.prepared = self.keys_as_values or self.whole_norm
+        if self.chunk is not None and (self.window or params.get("keep_first")):
+            raise ValueError("attention: a layer has a window or chunks, not both")
+        if self.keys_as_values and (self.shared_kv or v_dim != qk_dim):
+            raise ValueError("attention: keys serve as values in layers with keys of their own and "
+                             "values of their size")
+        if self.prepared and (params.get("conv") or params.get("query_temperature")
+                              or params.get("gate") or self.shared_kv or not self.keys_as_values
+                              or not self.whole_norm):
+            raise ValueError("attention: the norm over whole rows and keys that serve as values "
+                             "are built together, without convolutions, temperature, a gate per "
+                             "head or another layer's keys")
         # (heads, real size) of the projections this layer has, in the order of the row
         kinds = [("q", self.num_heads, qk_dim)]
         if not self.shared_kv:
-            kinds += [("k", self.num_kv_heads, qk_dim), ("v", self.num_kv_heads, v_dim)]
+            kinds.append(("k", self.num_kv_heads, qk_dim))
+            if not self.keys_as_values:
+                kinds.append(("v", self.num_kv_heads, v_dim))
         mats = [ctx.weights.pop(names[c]) for c, _, _ in kinds]
-        gate = ctx.weights.pop(join(prefix, params["gate"])) if params.get("gate") else None
+        gate_name = params.get("gate") or params.get("channel_gate")
+        gate = ctx.weights.pop(join(prefix, gate_name)) if gate_name else None
+        self.channel_gated = bool(params.get("channel_gate"))
         if len({t.dtype for t in mats + ([gate] if gate is not None else [])}) > 1:
             mats = [t.to(torch.float32) for t in mats]
             gate = None if gate is None else gate.to(torch.float32)
@@ -163,7 +201,17 @@ class PagedAttention(Mixer):
         # the columns of q, k and v in the product's rows
         self.qkv_cols = sum(t.shape[0] for t in mats)
         self.gated = gate is not None
-        if gate is not None:
+        if self.channel_gated:
+            # one gate per channel: the rows ride behind the others, from a multiple of 8 on
+            gate = self._pad_heads(gate, self.num_heads, v_dim, self.head_dim, rows=True)
+            lead = -self.qkv_cols % 8
+            if lead:
+                mats.append(gate.new_zeros((lead, gate.shape[1])))
+            mats.append(gate)
+            if gate.shape[0] % 8:
+                mats.append(gate.new_zeros((-gate.shape[0] % 8, gate.shape[1])))
+            self.gate_at = -(-self.qkv_cols // 8) * 8
+        elif gate is not None:
             # the gates' rows ride behind v, padded so that rows stay 16-byte aligned
             pad = -gate.shape[0] % 8
             mats.append(torch.cat([gate, gate.new_zeros((pad, gate.shape[1]))], dim=0))
@@ -178,12 +226,16 @@ class PagedAttention(Mixer):
                 for c, heads, size in kinds]).contiguous()
         self.q_norm = self.k_norm = None
         self.norm_eps = 0.0
-        norm = params.get("qk_norm")
         if norm:
             self.norm_eps = float(norm["eps"])
             self.q_norm = ctx.take(join(prefix, norm["q"])).to(torch.float32).contiguous()
             if not self.shared_kv:
                 self.k_norm = ctx.take(join(prefix, norm["k"])).to(torch.float32).contiguous()
+            if self.whole_norm:        # padded heads get zero weights
+                self.q_norm, self.k_norm = (
+                    self._pad_heads(t.reshape(-1, 1), heads, qk_dim, self.head_dim,
+                                    rows=True).reshape(-1).contiguous()
+                    for t, heads in ((self.q_norm, self.num_heads), (self.k_norm, self.num_kv_heads)))
         temp = params.get("query_temperature") or {}
         self.temp_coef, self.temp_every = float(temp.get("coef", 0.0)), int(temp.get("every", 0))
         self.sinks = None
@@ -233,12 +285,14 @@ class PagedAttention(Mixer):
             self.num_heads, self.num_kv_heads, self.head_dim, self.act_dtype,
             biased=getattr(self.position, "bias_slopes", None) is not None,
             shaped=self.head_scales is not None or self.softcap > 0,
-            plain=self.sinks is not None or bool(self.keep_first and self.window))
+            plain=self.sinks is not None or bool(self.keep_first and self.window),
+            span=self.chunk or 0)
 
     def cache_request(self) -> CacheRequest:
         if self.cache_like is not None:
             return CacheRequest.kv(self.num_kv_heads, self.head_dim, *self.cache_like)
-        return CacheRequest.kv(self.num_kv_heads, self.head_dim, self.window, self.keep_first)
+        return CacheRequest.kv(self.num_kv_heads, self.head_dim, self.window or self.chunk,
+                               self.keep_first)
 
     def step_planner(self):
         return self.planner
@@ -305,11 +359,13 @@ class PagedAttention(Mixer):
         if self.shared_kv and binding.writes:
             raise ValueError("attention: a layer without keys and values of its own must read "
                              "another run's cache")
-        rows = self._project(x, step, binding)
-        qkv = rows[:, :self.qkv_cols] if self.gated else rows
         if step.max_context > self.position.max_positions:
             raise ValueError(f"sequence of {step.max_context} positions exceeds max_seq_len "
                              f"{self.position.max_positions}")
+        if self.prepared:
+            return self._forward_prepared(x, step, binding, group)
+        rows = self._project(x, step, binding)
+        qkv = rows[:, :self.qkv_cols] if self.gated else rows
         out = ops.rope_attention(qkv, self.num_heads, self.num_kv_heads, self.head_dim,
                                  self.position.cos, self.position.sin, step.positions,
                                  group.slots, binding.k_pages, binding.v_pages, group.page_size,
@@ -320,7 +376,32 @@ class PagedAttention(Mixer):
                                  bias_slopes=getattr(self.position, "bias_slopes", None),
                                  counters=binding.counters, head_scales=self.head_scales,
                                  softcap=self.softcap, sinks=self.sinks,
-                                 keep_first=self.keep_first)
-        if self.gated:
+                                 keep_first=self.keep_first, chunk=self.chunk)
+        if self.channel_gated:
+            at = self.gate_at
+            ops.sigmoid_gate_(out, rows[:, at:at + out.shape[1]])
+        elif self.gated:
             ops.head_gate_(out, rows[:, self.qkv_cols:], self.num_heads, self.head_dim)
+        return ops.pending_linear(out, self.w_o, self.act_dtype)
+
+    def _forward_prepared(self, x: Any, step: Any, binding: CacheBinding, group: Any) -> Any:
+        """Layers whose keys serve as values behind norms over whole rows: one kernel adds the
+        biases, norms, rotates and lays out q, k and v; the attention kernels write k and v to
+        the cache as they come."""
+        rows = project(x, self.w_qkv, self.act_dtype)
+        pos = self.position
+        qkv = ops.row_prepare(rows, self.num_heads, self.num_kv_heads, self.head_dim, self.qk_dim,
+                              self.bias, self.q_norm, self.k_norm, self.norm_eps, pos.cos, pos.sin,
+                              step.positions, bool(getattr(pos, "interleaved", False)))
+        out = ops.rope_attention(qkv, self.num_heads, self.num_kv_heads, self.head_dim, None, None,
+                                 step.positions, group.slots, binding.k_pages, binding.v_pages,
+                                 group.page_size, group.block_tables, step, self.scale, self.window,
+                                 write_kv=binding.writes, plan=step.plans.get(self.planner.key()),
+                                 bias_slopes=getattr(pos, "bias_slopes", None),
+                                 counters=binding.counters, head_scales=self.head_scales,
+                                 softcap=self.softcap, sinks=self.sinks,
+                                 keep_first=self.keep_first, chunk=self.chunk)
+        if self.channel_gated:
+            at = self.gate_at
+            ops.sigmoid_gate_(out, rows[:, at:at + out.shape[1]])
         return ops.pending_linear(out, self.w_o, self.act_dtype)

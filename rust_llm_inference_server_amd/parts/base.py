@@ -243,6 +243,14 @@ class Norm(Part):
     def forward_rows(self, stream: "ResidualStream", rows: torch.Tensor) -> torch.Tensor:
         raise NotImplementedError
 
+    def join(self, stream: "ResidualStream", delta: torch.Tensor,
+             out_dtype: Optional[torch.dtype]) -> Optional[torch.Tensor]:
+        """``x += norm(delta)`` in the 32-bit residual (``delta`` whole, or a stack of float32
+        partial sums); returns the new residual in ``out_dtype`` (None: nothing).  For blocks
+        whose norms stand behind their sublayers; a norm that has no such kernel has no such
+        use."""
+        raise NotImplementedError
+
     def fused_linear(self, stream: "ResidualStream", w: torch.Tensor, out_dtype: torch.dtype,
                      gated: bool, rows: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
         """The norm and the projection behind it in one kernel: ``norm(stream) @ w.T`` (gated:
@@ -347,9 +355,16 @@ class Block(Part):
 
 
 class Embedding(Part):
+    # True when forward also takes the step and the part's binding (``forward(ids, positions,
+    # step=..., binding=...)``): a part that looks at earlier tokens or keeps state per request.
+    wants_step = False
     # positions the part can place (a table of learned position vectors has so many rows);
     # None: any
     position_rows: Optional[int] = None
+
+    def state_bytes(self) -> int:
+        """Bytes of fixed-size state the part keeps per request (as for a mixer)."""
+        return 0
 
     def forward(self, ids: torch.Tensor, positions: Optional[torch.Tensor] = None) -> torch.Tensor:
         """Token ids ``(T)`` int32 (and their absolute positions ``(T)`` int32, for a part that
@@ -437,7 +452,8 @@ class ResidualStream:
     (``round_parts``), as a delta that arrives whole in bfloat16 was by its kernel, so that the
     rounding does not depend on which kernel a batch's size chose."""
 
-    __slots__ = ("x", "pending", "pending_scale", "round_parts", "history", "lanes")
+    __slots__ = ("x", "pending", "pending_scale", "pending_norm", "round_parts", "history",
+                 "lanes", "act_dtype")
 
     def __init__(self, x: torch.Tensor, act_dtype: torch.dtype = torch.float32):
         assert x.dtype == torch.float32
@@ -448,6 +464,10 @@ class ResidualStream:
         # the multiplier with which the pending delta joins the sum (in float32, by whoever
         # adds it); a norm's fused forms take deltas with multiplier 1 only
         self.pending_scale = 1.0
+        # the norm that the pending delta passes on its way into the sum (blocks whose norms
+        # stand behind their sublayers); such a delta is folded in by ``rows`` or ``flush``
+        self.pending_norm: Optional[Norm] = None
+        self.act_dtype = act_dtype
         self.round_parts = act_dtype == torch.bfloat16
         # (slots, T, H) float32: the embedding output and the layers' results so far, for
         # blocks that feed the next layer a mix of them (made by the first such block)
@@ -470,26 +490,46 @@ class ResidualStream:
         if self.lanes is not None:
             self.x, self.lanes = self.lanes.total(), None
 
-    def add(self, delta: Any, scale: float = 1.0) -> None:
+    def add(self, delta: Any, scale: float = 1.0, norm: Optional[Norm] = None) -> None:
         if self.pending is not None:
             self.flush()
         self.pending = delta
         self.pending_scale = float(scale)
+        self.pending_norm = norm
+
+    def rows(self) -> torch.Tensor:
+        """The residual itself (a pending delta folded in) in the activation dtype, for
+        sublayers without a norm in front."""
+        from .. import ops
+        norm, self.pending_norm = self.pending_norm, None
+        if norm is None:
+            self.flush()
+            return ops.norm_join(self.x, None, None, 0.0, self.act_dtype)
+        delta, self.pending = self.delta(), None
+        return norm.join(self, delta, self.act_dtype)
 
     def take_delta(self) -> Tuple[Optional[torch.Tensor], float]:
         """The pending delta as a tensor with its multiplier; the stream then has none."""
+        if self.pending_norm is not None:
+            self.flush()
         delta, scale = self.delta(), self.pending_scale
         self.pending, self.pending_scale = None, 1.0
         return delta, scale
 
     def delta(self) -> Optional[torch.Tensor]:
         """The pending delta as a tensor (a product that has not run yet runs now)."""
+        if self.pending_norm is not None:
+            self.flush()
         if self.pending is not None and not isinstance(self.pending, torch.Tensor):
             self.pending = self.pending.run()
         return self.pending
 
     def flush(self) -> torch.Tensor:
         """Fold a pending delta into the residual and return the residual."""
+        if self.pending is not None and self.pending_norm is not None:
+            norm, self.pending_norm = self.pending_norm, None
+            delta, self.pending = self.delta(), None
+            norm.join(self, delta, None)
         if self.pending is not None:
             from .. import ops
             ops.add_residual(self.x, self.delta(), round_parts=self.round_parts,

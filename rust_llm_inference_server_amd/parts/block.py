@@ -1,5 +1,6 @@
 """Decoder blocks.  The pre-norm block: ``x += mixer(norm(x)); x += feed_forward(norm(x))``
-(crates/model/src/llama.rs:264-271).  Which mixer, feed-forward and norms it holds, and under
+(crates/model/src/llama.rs:264-271).  The post-norm block: ``x += norm(mixer(x)); x +=
+norm(feed_forward(x))``.  Which mixer, feed-forward and norms it holds, and under
 which weight names, is given by its parameters, layer by layer.  The parallel block:
 ``x += mixer(h) + feed_forward(h)`` with ``h = norm(x)``, one norm that both sublayers read, or
 ``x += mixer(norm(x)) + feed_forward(ffn_norm(x))`` with a norm each of the same x.  Behind
@@ -118,6 +119,58 @@ class HyperBlock(PreNormBlock):
         lanes.reading(None)          # whoever reads next without weights reads the plain sum
         if self.last:
             stream.merge_lanes()
+
+
+@register("block", "postnorm")
+class PostNormBlock(Block):
+    """Norms behind the sublayers: ``x += mixer_norm(mixer(x)); x += ffn_norm(ff(x))``, the
+    sublayers reading x itself, and optionally a third sublayer of a token's own input,
+    ``x += side_norm(side(x))``.
+
+    Parameters: ``mixer``, ``mixer_norm``, ``feed_forward`` and ``ffn_norm``, ``side`` and
+    ``side_norm`` (PartSpecs; ``feed_forward`` and ``side``, both feed-forward kinds, may be None)
+    and ``names``: the weight-name suffix of each under the block's prefix.  A sublayer's result
+    is left pending; one kernel norms it, adds it to the float32 stream and leaves the stream in
+    the activation dtype for the next sublayer to read."""
+
+    _SLOTS = (("mixer_norm", "norm"), ("mixer", "mixer"), ("ffn_norm", "norm"),
+              ("feed_forward", "feed_forward"), ("side_norm", "norm"), ("side", "feed_forward"))
+
+    @classmethod
+    def _slots(cls, params: Dict[str, Any]):
+        gone = set()
+        if params.get("feed_forward") is None:
+            gone |= {"feed_forward", "ffn_norm"}
+        if params.get("side") is None:
+            gone |= {"side", "side_norm"}
+        return [(slot, category) for slot, category in cls._SLOTS if slot not in gone]
+
+    @classmethod
+    def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
+        out: List[TensorSpec] = []
+        for slot, category in cls._slots(params):
+            out += tensor_specs(category, params[slot], join(prefix, params["names"][slot]))
+        return out
+
+    def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
+        super().__init__(params, prefix, ctx)
+        built = {slot: create(category, params[slot], join(prefix, params["names"][slot]), ctx)
+                 for slot, category in self._slots(params)}
+        self.mixer, self.mixer_norm = built["mixer"], built["mixer_norm"]
+        self.feed_forward, self.ffn_norm = built.get("feed_forward"), built.get("ffn_norm")
+        self.side, self.side_norm = built.get("side"), built.get("side_norm")
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(p.graph_safe for p in (self.mixer, self.mixer_norm, self.feed_forward,
+                                          self.ffn_norm, self.side, self.side_norm)
+                   if p is not None)
+
+    def forward(self, stream: ResidualStream, step: Any, binding: CacheBinding) -> None:
+        stream.add(self.mixer.forward(stream.rows(), step, binding), norm=self.mixer_norm)
+        for part, norm in ((self.feed_forward, self.ffn_norm), (self.side, self.side_norm)):
+            if part is not None:
+                stream.add(part.forward(stream.rows(), step), norm=norm)
 
 
 @register("block", "parallel")

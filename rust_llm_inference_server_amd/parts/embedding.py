@@ -18,9 +18,14 @@ from .base import BuildContext, Embedding, Head, TensorSpec, join, project, regi
 class TokenEmbedding(Embedding):
     """Parameters: ``vocab_size``, ``hidden_size``; optional ``scale`` (the rows are multiplied
     by it as they enter the float32 stream), ``weight_name`` (the table's name under the
-    prefix, "weight" by default; "" when it is stored under the prefix itself) and
+    prefix, "weight" by default; "" when it is stored under the prefix itself),
     ``learned_positions``: ``{"name": full tensor name, "rows": positions}``, a table of
-    learned position vectors of which row p is added, unscaled, to the token at position p."""
+    learned position vectors of which row p is added, unscaled, to the token at position p, and
+    ``bigram``: ``{"name": full tensor name, "buckets": n, "mul_prev": a, "mul_cur": b}``, a
+    table of n + 1 rows of which row ``(a previous + b token) mod n`` is added, unscaled, to a
+    token behind another one, and the last row to a sequence's first token.  The previous token
+    of a portion's first token comes from the request's state slot, where every step leaves the
+    last token it brought."""
 
     graph_safe = True
 
@@ -31,6 +36,9 @@ class TokenEmbedding(Embedding):
         learned = params.get("learned_positions")
         if learned:
             out.append(TensorSpec(learned["name"], (learned["rows"], params["hidden_size"])))
+        bigram = params.get("bigram")
+        if bigram:
+            out.append(TensorSpec(bigram["name"], (bigram["buckets"] + 1, params["hidden_size"])))
         return out
 
     def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
@@ -47,8 +55,31 @@ class TokenEmbedding(Embedding):
                 self.learned = self.learned.to(torch.float32).contiguous()
                 self.weight = self.weight.to(torch.float32).contiguous()
             self.position_rows = int(self.learned.shape[0])
+        self.bigram = None
+        bigram = params.get("bigram")
+        if bigram:
+            if self.learned is not None:
+                raise ValueError("embedding: a table of pairs beside learned positions is not built")
+            self.wants_step = True
+            self.bigram = ctx.take(bigram["name"])
+            if self.bigram.dtype != self.weight.dtype:
+                self.bigram = self.bigram.to(torch.float32).contiguous()
+                self.weight = self.weight.to(torch.float32).contiguous()
+            self.mul_prev, self.mul_cur = int(bigram["mul_prev"]), int(bigram["mul_cur"])
 
-    def forward(self, ids: torch.Tensor, positions: Any = None) -> torch.Tensor:
+    def state_bytes(self) -> int:
+        """The last token of the request, plus one (int32; 0: there is none yet)."""
+        return 0 if self.bigram is None else 4
+
+    def forward(self, ids: torch.Tensor, positions: Any = None, step: Any = None,
+                binding: Any = None) -> torch.Tensor:
+        if self.bigram is not None:
+            if binding is None or binding.state is None:
+                raise ValueError("embedding: the table of pairs needs a state slot per request; "
+                                 "the runner has none")
+            return ops.embed_pairs(ids, self.weight, self.scale, self.bigram, self.mul_prev,
+                                   self.mul_cur, binding.state.view(torch.int32),
+                                   step.seq_of_token, step.cu_seqlens, step.state_slots)
         if self.learned is None:
             return ops.embed(ids, self.weight, self.scale)
         if positions is None:

@@ -84,6 +84,77 @@ class DenseMLP(FeedForward):
         return ops.pending_linear(hidden, self.w_down, self.act_dtype)
 
 
+@register("feed_forward", "gated_mlp")
+class GatedMLP(FeedForward):
+    """A gated unit, ``down(act(gate(x)) * up(x))``, three bias-free projections, gate and up as
+    one product over the row-concatenated weights.
+
+    Parameters: ``hidden_size``, ``intermediate_size``, ``activation`` ("gelu_tanh"), ``names``
+    (the tensors of gate, up and down under the prefix)."""
+
+    graph_safe = True
+
+    @classmethod
+    def _names(cls, params: Dict[str, Any], prefix: str) -> Dict[str, str]:
+        return {k: join(prefix, v) for k, v in params["names"].items()}
+
+    @classmethod
+    def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
+        H, I = params["hidden_size"], params["intermediate_size"]
+        n = cls._names(params, prefix)
+        return [TensorSpec(n["gate"], (I, H)), TensorSpec(n["up"], (I, H)),
+                TensorSpec(n["down"], (H, I))]
+
+    def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
+        super().__init__(params, prefix, ctx)
+        if params.get("activation", "gelu_tanh") != "gelu_tanh":
+            raise ValueError(f"feed-forward 'gated_mlp': activation '{params['activation']}' is not "
+                             "known (known: 'gelu_tanh'; 'swiglu' is a kind of its own)")
+        n = self._names(params, prefix)
+        gate, up = ctx.weights.pop(n["gate"]), ctx.weights.pop(n["up"])
+        if gate.dtype != up.dtype:
+            gate, up = gate.to(torch.float32), up.to(torch.float32)
+        self.w_gate_up = torch.cat([gate, up], dim=0).contiguous()
+        del gate, up
+        self.w_down = ctx.take(n["down"])
+        self.act_dtype = ctx.act_dtype
+
+    def forward(self, x: torch.Tensor, step: Any) -> Any:
+        hidden = ops.linear_geglu(x, self.w_gate_up)
+        return ops.pending_linear(hidden, self.w_down, self.act_dtype)
+
+
+@register("feed_forward", "token_side")
+class TokenSide(FeedForward):
+    """A layer's own token input: ``proj(gelu(gate(x)) * e)`` with ``e`` this layer's part of the
+    token's row in a second embedding table (columns ``index * dim`` to ``(index + 1) * dim``),
+    the tanh form of GELU.
+
+    Parameters: ``hidden_size``, ``vocab_size``, ``dim``, ``index`` (the layer's part), ``parts``
+    (parts of a row), ``table`` (the table's full tensor name, ``(vocab_size, parts * dim)``;
+    all layers share it).  Tensors under the prefix: ``gate`` (dim, W), ``proj`` (W, dim)."""
+
+    graph_safe = True
+
+    @classmethod
+    def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
+        W, d = params["hidden_size"], params["dim"]
+        return [TensorSpec(params["table"], (params["vocab_size"], params["parts"] * d), std=1.0),
+                TensorSpec(join(prefix, "gate"), (d, W)), TensorSpec(join(prefix, "proj"), (W, d))]
+
+    def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
+        super().__init__(params, prefix, ctx)
+        self.dim, self.index = int(params["dim"]), int(params["index"])
+        self.table = ctx.take(params["table"])
+        self.w_gate, self.w_proj = ctx.take(join(prefix, "gate")), ctx.take(join(prefix, "proj"))
+        self.act_dtype = ctx.act_dtype
+
+    def forward(self, x: torch.Tensor, step: Any) -> Any:
+        z = ops.linear(x, self.w_gate, self.act_dtype)
+        g = ops.side_gate_(z, self.table, self.index * self.dim, step.ids)
+        return ops.pending_linear(g, self.w_proj, self.act_dtype)
+
+
 @register("feed_forward", "clamped_glu")
 class ClampedGLU(FeedForward):
     """A gated unit whose branches are bounded before they meet:

@@ -64,10 +64,17 @@ class RMSNorm(Norm):
                                rows=rows, round_parts=stream.round_parts,
                                delta_scale=stream.pending_scale)
 
+    def join(self, stream: ResidualStream, delta: torch.Tensor,
+             out_dtype: Optional[torch.dtype]) -> Optional[torch.Tensor]:
+        return ops.norm_join(stream.x, delta, self.weight, self.eps, out_dtype,
+                             round_parts=stream.round_parts)
+
     def fused_linear(self, stream: ResidualStream, w: torch.Tensor, out_dtype: torch.dtype,
                      gated: bool, rows: Optional[torch.Tensor]) -> Optional[torch.Tensor]:
         if self.out_dtype != torch.bfloat16 or stream.lanes is not None:
             return None
+        if stream.pending_norm is not None:
+            stream.flush()
         if stream.pending is not None and stream.pending_scale != 1.0:
             if rows is not None:
                 return None

@@ -24,6 +24,14 @@ numbers per channel decays by ``exp(dt A)`` with a step ``dt`` that the token ch
 head ``S <- decay_h S + k v^T`` and the read-out ``S^T q`` includes the token's own key and
 value; the heads' read-outs are normalised together, gated by a sigmoid and projected.
 
+``channel_delta``: the gated delta rule with one decay per head and key channel (a low-rank
+projection of the token's input), a write that its own token already reads, and a sigmoid gate
+(low-rank too) behind the heads' norm.
+
+``rglru`` (a real-gated linear recurrent unit): one number per channel behind a short
+convolution decays by ``a = exp(-c r softplus(lam))`` and takes ``sqrt(1 - a^2) i u``, the gates r
+and i being block-diagonal products of u; the result meets a GELU branch of the input.
+
 ``parallel``: two mixers read the same input, and their outputs meet as a weighted sum in
 float32.  Each keeps what it keeps: the pages of the one that asks for a cache, the state
 bytes of both, one after the other.
@@ -361,6 +369,199 @@ class DecayAttention(Mixer):
                                 H, d, dv, longest=getattr(step, "max_new", None))
         y = ops.head_norm_gate(o, self.norm, p[:, c["g"]:c["g"] + H * dv], 1, H * dv, self.eps,
                                self.act_dtype, sigmoid_gate=True)
+        return ops.pending_linear(y, self.w_o, self.act_dtype)
+
+
+# -------------------------------------------------------------------------- channel delta
+@register("mixer", "channel_delta")
+class ChannelDelta(Mixer):
+    """Parameters: ``hidden_size``, ``num_heads`` (value heads), ``num_kv_heads`` (query/key
+    heads; value head h uses head ``h // (heads / kv_heads)``), ``head_dim``, ``value_dim``,
+    ``conv`` (taps), ``decay_rank``, ``gate_rank``, ``eps`` (of the per-head norm of the read-out).
+
+    Tensors under the prefix: ``q``, ``k`` (kv_heads * d, W), ``v`` (heads * dv, W), each with
+    ``.conv`` (channels, taps); ``b`` (heads, W); ``A_log`` (heads); ``a1`` (decay_rank, W), ``a2``
+    (heads * d, decay_rank), ``dt_bias`` (heads * d); ``g1`` (gate_rank, W), ``g2`` (heads * dv,
+    gate_rank); ``norm`` (dv); ``o`` (W, heads * dv).
+
+    Per token and head, with ``g = exp(-exp(A_log) softplus(a2 (a1 h) + dt_bias))`` per key
+    channel: ``S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q``, ``beta =
+    sigmoid(b h)``, q and k unit vectors behind convolution and SiLU, q times ``d^-1/2``.
+
+    One product makes q, k, v and b (stored float32); the two low-rank pairs share two products:
+    ``[a1; g1]`` and the block-diagonal ``[a2 0; 0 g2]``."""
+
+    graph_safe = True
+    UNIT_EPS = 1e-6
+
+    @classmethod
+    def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
+        W, H, G = params["hidden_size"], params["num_heads"], params["num_kv_heads"]
+        d, dv, taps = params["head_dim"], params["value_dim"], params["conv"]
+        ra, rg = params["decay_rank"], params["gate_rank"]
+        out = []
+        for n, rows in (("q", G * d), ("k", G * d), ("v", H * dv)):
+            out += [TensorSpec(join(prefix, n), (rows, W)),
+                    TensorSpec(join(prefix, f"{n}.conv"), (rows, taps), std=0.3)]
+        out += [TensorSpec(join(prefix, "b"), (H, W)), TensorSpec(join(prefix, "A_log"), (H,)),
+                TensorSpec(join(prefix, "norm"), (dv,), init="ones_normal"),
+                TensorSpec(join(prefix, "a1"), (ra, W)), TensorSpec(join(prefix, "a2"), (H * d, ra)),
+                TensorSpec(join(prefix, "dt_bias"), (H * d,)),
+                TensorSpec(join(prefix, "g1"), (rg, W)), TensorSpec(join(prefix, "g2"), (H * dv, rg)),
+                TensorSpec(join(prefix, "o"), (W, H * dv))]
+        return out
+
+    def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
+        super().__init__(params, prefix, ctx)
+        self.width = int(params["hidden_size"])
+        self.heads, self.kv_heads = int(params["num_heads"]), int(params["num_kv_heads"])
+        self.dim, self.vdim = int(params["head_dim"]), int(params["value_dim"])
+        self.taps = int(params["conv"])
+        self.eps = float(params["eps"])
+        if self.heads % self.kv_heads:
+            raise ValueError(f"channel_delta: {self.heads} heads are not a multiple of "
+                             f"{self.kv_heads} query/key heads")
+        if not 1 <= self.taps <= 16:
+            raise ValueError(f"channel_delta: {self.taps} taps (1 to 16)")
+        if self.dim > 256:
+            raise ValueError(f"channel_delta: heads of {self.dim} key channels (at most 256)")
+        pop = lambda n: ctx.weights.pop(join(prefix, n))
+        take = lambda n: ctx.take(join(prefix, n))
+        G, H, d, dv = self.kv_heads, self.heads, self.dim, self.vdim
+        self.conv_channels = C = 2 * G * d + H * dv
+        parts = [pop("q"), pop("k"), pop("v"), pop("b")]
+        if len({p.dtype for p in parts}) > 1:
+            parts = [p.to(torch.float32) for p in parts]
+        # columns of the product: q | k | v | b, b from a multiple of 8
+        self.b_at = -(-C // 8) * 8
+        rows = parts[:3]
+        if self.b_at > C:
+            rows.append(parts[0].new_zeros((self.b_at - C, self.width)))
+        rows.append(parts[3])
+        if H % 8:
+            rows.append(parts[0].new_zeros((-H % 8, self.width)))
+        self.w_in = torch.cat(rows, dim=0).contiguous()
+        del parts, rows
+        self.conv_w = torch.cat([_f32(take(f"{n}.conv")) for n in "qkv"], dim=0).contiguous()
+        a1, g1, a2, g2 = pop("a1"), pop("g1"), pop("a2"), pop("g2")
+        if len({p.dtype for p in (a1, g1, a2, g2)}) > 1:
+            a1, g1, a2, g2 = (p.to(torch.float32) for p in (a1, g1, a2, g2))
+        ra, rg = a1.shape[0], g1.shape[0]
+        at = -(-ra // 8) * 8
+        self.w_low = a1.new_zeros((at + -(-rg // 8) * 8, self.width))
+        self.w_low[:ra], self.w_low[at:at + rg] = a1, g1
+        # (the second product's gate columns start on a multiple of 8 too)
+        self.gate_at = -(-H * d // 8) * 8
+        self.w_up = a2.new_zeros((self.gate_at + H * dv, self.w_low.shape[0]))
+        self.w_up[:H * d, :ra], self.w_up[self.gate_at:, at:at + rg] = a2, g2
+        self.a_log, self.dt_bias = _f32(take("A_log")), _f32(take("dt_bias"))
+        self.norm = _f32(take("norm"))
+        self.w_o = take("o")
+        self.act_dtype = ctx.act_dtype
+
+    def state_bytes(self) -> int:
+        return 4 * ((self.taps - 1) * self.conv_channels + self.heads * self.vdim * self.dim)
+
+    def forward(self, x: torch.Tensor, step: Any, binding: CacheBinding) -> Any:
+        G, H, d, dv, C = self.kv_heads, self.heads, self.dim, self.vdim, self.conv_channels
+        tail, S = _state_views(binding, (self.taps - 1) * C)
+        cu, slots, n = step.cu_seqlens, step.state_slots, step.num_seqs
+        p = ops.linear_f32(x, self.w_in)                                   # (T, q|k|v|b)
+        up = ops.linear_f32(ops.linear(x, self.w_low, self.act_dtype), self.w_up)
+        qkv = ops.causal_conv(p, self.conv_w, tail, step.seq_of_token, cu, slots, n,
+                              unit_channels=2 * G * d, unit_group=d, scaled_channels=G * d,
+                              scale=d ** -0.5, unit_eps=self.UNIT_EPS, rest_group=min(dv, 1024))
+        ops.tail_update(tail, p, C, self.taps - 1, cu, slots, n)
+        o = ops.channel_delta_scan(qkv[:, :G * d], qkv[:, G * d:2 * G * d], qkv[:, 2 * G * d:],
+                                   p[:, self.b_at:self.b_at + H], up[:, :H * d], self.a_log,
+                                   self.dt_bias, S, cu, slots, n, H, G, d, dv)
+        y = ops.head_norm_gate(o, self.norm, up[:, self.gate_at:], H, dv, self.eps, self.act_dtype,
+                               sigmoid_gate=True)
+        return ops.pending_linear(y, self.w_o, self.act_dtype)
+
+
+# --------------------------------------------------------- real-gated linear recurrent unit
+@register("mixer", "rglru")
+class RGLRU(Mixer):
+    """Parameters: ``hidden_size``, ``width`` (channels), ``blocks`` (equal parts of the channels
+    that the gates' products stay inside), ``conv`` (taps), ``power`` (the factor in the log
+    decay).
+
+    Tensors under the prefix: ``y``, ``x`` (width, W) with ``.b`` (width); ``conv`` (width, taps)
+    and ``conv.b``; ``ra``, ``ri`` (blocks, n, n), each [out, in], with ``.b`` (blocks, n);
+    ``lam`` (width); ``o`` (W, width).
+
+    Per token and channel: ``u = conv(x h + x.b)`` (zeros in front of the sequence), ``r, i =
+    sigmoid(ra u + ra.b), sigmoid(ri u + ri.b)`` block by block, ``log a = -power r
+    softplus(lam)``, ``S <- a S + sqrt(1 - a^2) i u``, result ``S gelu(y h + y.b)`` (tanh form).
+    The state slot holds the last ``conv - 1`` inputs of the convolution and S, float32."""
+
+    graph_safe = True
+
+    @classmethod
+    def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
+        W, C, B, taps = (params[k] for k in ("hidden_size", "width", "blocks", "conv"))
+        n = C // B
+        out = []
+        for name in ("y", "x"):
+            out += [TensorSpec(join(prefix, name), (C, W)), TensorSpec(join(prefix, name + ".b"), (C,))]
+        out += [TensorSpec(join(prefix, "conv"), (C, taps), std=0.3),
+                TensorSpec(join(prefix, "conv.b"), (C,))]
+        for name in ("ra", "ri"):
+            out += [TensorSpec(join(prefix, name), (B, n, n)),
+                    TensorSpec(join(prefix, name + ".b"), (B, n))]
+        return out + [TensorSpec(join(prefix, "lam"), (C,), std=0.5),
+                      TensorSpec(join(prefix, "o"), (W, C))]
+
+    def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
+        super().__init__(params, prefix, ctx)
+        self.width = int(params["hidden_size"])
+        self.channels, self.blocks = int(params["width"]), int(params["blocks"])
+        self.taps, self.power = int(params["conv"]), float(params["power"])
+        if self.channels % self.blocks:
+            raise ValueError(f"rglru: {self.channels} channels in {self.blocks} blocks")
+        if not 1 <= self.taps <= 16:
+            raise ValueError(f"rglru: {self.taps} taps (1 to 16)")
+        pop = lambda n: ctx.weights.pop(join(prefix, n))
+        take = lambda n: ctx.take(join(prefix, n))
+        C = self.channels
+        wx, wy = pop("x"), pop("y")
+        if wx.dtype != wy.dtype:
+            wx, wy = wx.to(torch.float32), wy.to(torch.float32)
+        # columns of the one product: x | y, y from a multiple of 8
+        self.y_at = -(-C // 8) * 8
+        rows = [wx] + ([wx.new_zeros((self.y_at - C, self.width))] if self.y_at > C else []) + [wy]
+        self.w_in = torch.cat(rows, dim=0).contiguous()
+        del wx, wy, rows
+        self.x_bias, self.y_bias = _f32(take("x.b")), _f32(take("y.b"))
+        self.conv_w, self.conv_b = _f32(take("conv")), _f32(take("conv.b"))
+        # per block the rows of ra in front of those of ri
+        self.w_gates = torch.cat([pop("ra").to(ctx.act_dtype), pop("ri").to(ctx.act_dtype)],
+                                 dim=1).contiguous()
+        self.r_bias = _f32(take("ra.b")).reshape(-1).contiguous()
+        self.i_bias = _f32(take("ri.b")).reshape(-1).contiguous()
+        # -power softplus(lam), float32, made once
+        self.rate = (-self.power * torch.nn.functional.softplus(
+            take("lam").to(torch.float64), threshold=40.0)).to(torch.float32).contiguous()
+        self.w_o = take("o")
+        self.act_dtype = ctx.act_dtype
+
+    def state_bytes(self) -> int:
+        return 4 * self.taps * self.channels
+
+    def forward(self, x: torch.Tensor, step: Any, binding: CacheBinding) -> Any:
+        C, n = self.channels, self.channels // self.blocks
+        tail, S = _state_views(binding, (self.taps - 1) * C)
+        cu, slots, num = step.cu_seqlens, step.state_slots, step.num_seqs
+        p = ops.linear_f32(x, self.w_in)                                   # (T, x | y)
+        u = ops.causal_conv(p, self.conv_w, tail, step.seq_of_token, cu, slots, num,
+                            bias=self.conv_b, out_dtype=self.act_dtype, activation=False,
+                            in_bias=self.x_bias)
+        ops.tail_update(tail, p, C, self.taps - 1, cu, slots, num, bias=self.x_bias)
+        gates = ops.head_linear(u, self.w_gates, n, out_dtype=torch.float32)
+        y = ops.rglru_scan(u, gates, self.r_bias, self.i_bias, self.rate,
+                           p[:, self.y_at:self.y_at + C], self.y_bias, S, cu, slots, num,
+                           self.blocks, longest=getattr(step, "max_new", None))
         return ops.pending_linear(y, self.w_o, self.act_dtype)
 
 

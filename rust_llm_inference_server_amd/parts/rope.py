@@ -47,17 +47,21 @@ def inverse_frequencies(rot_dim: int, theta: float, scaling: Optional[Dict[str, 
     f32 = torch.float32
     exponent = torch.arange(0, rot_dim, 2, dtype=f32) / torch.tensor(float(rot_dim), dtype=f32)
     inv = 1.0 / torch.pow(torch.tensor(float(theta), dtype=f32), exponent)
-    if not scaling:
-        return inv
+    return llama3_scaled(inv, scaling) if scaling else inv
+
+
+def llama3_scaled(inv: torch.Tensor, scaling: Dict[str, Any]) -> torch.Tensor:
+    """The frequencies under the llama3 rule, in the precision they come in."""
+    dt = inv.dtype
     kind = scaling.get("rope_type")
     if kind != "llama3":
         raise ValueError(f"position encoding 'rope': unknown scaling '{kind}' (known: 'llama3')")
-    factor = torch.tensor(float(scaling["factor"]), dtype=f32)
-    low = torch.tensor(float(scaling["low_freq_factor"]), dtype=f32)
-    high = torch.tensor(float(scaling["high_freq_factor"]), dtype=f32)
-    old_ctx = torch.tensor(float(scaling["original_max_position_embeddings"]), dtype=f32)
+    factor = torch.tensor(float(scaling["factor"]), dtype=dt)
+    low = torch.tensor(float(scaling["low_freq_factor"]), dtype=dt)
+    high = torch.tensor(float(scaling["high_freq_factor"]), dtype=dt)
+    old_ctx = torch.tensor(float(scaling["original_max_position_embeddings"]), dtype=dt)
     low_wavelen, high_wavelen = old_ctx / low, old_ctx / high
-    wavelen = torch.tensor(2.0 * math.pi, dtype=f32) / inv
+    wavelen = torch.tensor(2.0 * math.pi, dtype=dt) / inv
     smooth = (old_ctx / wavelen - low) / (high - low)
     blended = (1.0 - smooth) * inv / factor + smooth * inv
     return torch.where(wavelen < high_wavelen, inv,
@@ -70,6 +74,7 @@ class RotaryEmbedding(PositionEncoding):
     (None, the llama3 fields, ``{"rope_type": "yarn", "factor", "original", "fast",
     "slow"}``, or with ``precise`` ``{"rope_type": "linear", "factor"}``: every frequency divided
     by the factor).  Holds ``cos``/``sin`` float32 ``(max_positions, rot/2)``.
+    Optional ``interleaved``: the rotation pairs dim 2j with 2j + 1 instead of j with j + rot/2.
     Optional ``precise``: frequencies, angles, cosines and sines are made in double precision
     and rounded once to float32 (without it they are float32 from the start, as the reference
     makes them); yarn scaling is always made that way."""
@@ -86,11 +91,14 @@ class RotaryEmbedding(PositionEncoding):
             magnitude = 0.1 * math.log(float(scaling["factor"])) + 1.0
             pos = torch.arange(ctx.max_positions, dtype=torch.float64).reshape(-1, 1)
         elif params.get("precise"):
-            if scaling and scaling.get("rope_type") != "linear":
-                raise ValueError("position encoding 'rope': 'precise' has no llama3 scaling")
+            kind = scaling.get("rope_type") if scaling else None
+            if kind not in (None, "linear", "llama3"):
+                raise ValueError(f"position encoding 'rope': unknown scaling '{kind}'")
             f64 = torch.float64
             inv = float(params["theta"]) ** (-torch.arange(0, rot, 2, dtype=f64) / rot)
-            if scaling:
+            if kind == "llama3":
+                inv = llama3_scaled(inv, scaling)
+            elif kind == "linear":
                 # positions stretched evenly: every frequency divided by the factor
                 factor = float(scaling.get("factor") or 0.0)
                 if not factor > 0:
@@ -103,6 +111,7 @@ class RotaryEmbedding(PositionEncoding):
             pos = torch.arange(ctx.max_positions, dtype=torch.float32).reshape(-1, 1)
         angles = pos * inv.reshape(1, -1)
         self.rot_dim = rot
+        self.interleaved = bool(params.get("interleaved"))
         self.inv_freq = inv.to(torch.float32)
         self.cos = (torch.cos(angles) * magnitude).to(torch.float32).to(ctx.device).contiguous()
         self.sin = (torch.sin(angles) * magnitude).to(torch.float32).to(ctx.device).contiguous()

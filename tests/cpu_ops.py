@@ -27,6 +27,62 @@ def gelu_erf(x):
     return (0.5 * z * (1.0 + torch.erf(z * 0.7071067811865476))).to(x.dtype)
 
 
+def geglu(gu):
+    i = gu.shape[1] // 2
+    return (gelu_tanh(gu[:, :i].float()) * gu[:, i:].float()).to(gu.dtype)
+
+
+def linear_geglu(x, w_gate_up):
+    return geglu(linear(x, w_gate_up, x.dtype))
+
+
+def norm_join(resid, y, weight, eps, out_dtype=None, round_parts=False):
+    if y is not None:
+        y = (y.sum(0) if y.dim() == 3 else y).float()
+        resid += y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps) * weight.float()
+    return None if out_dtype is None else resid.to(out_dtype)
+
+
+def side_gate_(z, table, column, ids):
+    e = table[ids.long()][:, column:column + z.shape[1]]
+    z.copy_((gelu_tanh(z.float()) * e.float()).to(z.dtype))
+    return z
+
+
+def embed_pairs(ids, table, scale, pairs, mul_prev, mul_cur, last, seq_of_token, cu, slots):
+    n = pairs.shape[0] - 1
+    rows = []
+    ids_l = ids.tolist()
+    for t0, t1, slot in _seqs(cu, slots, cu.numel() - 1):
+        before = int(last[slot, 0]) - 1
+        for t in range(t0, t1):
+            rows.append(n if before < 0 else (before * mul_prev + ids_l[t] * mul_cur) % n)
+            before = ids_l[t]
+        last[slot, 0] = before + 1
+    return table[ids.long()].float() * scale + pairs[torch.tensor(rows)].float()
+
+
+def row_prepare(p, num_heads, num_kv_heads, head_dim, real_dim, bias, q_weight, k_weight, eps, cos,
+                sin, positions, interleaved=False):
+    assert interleaved or cos is None, "the test double rotates neighbouring dims only"
+    T, nh, nkv, D = p.shape[0], num_heads, num_kv_heads, head_dim
+    x = p[:, :(nh + nkv) * D].float()
+    if bias is not None:
+        x = x + bias
+    v = x[:, nh * D:]
+    out = []
+    for part, heads, w in ((x[:, :nh * D], nh, q_weight), (v, nkv, k_weight)):
+        ms = (part * part).sum(-1, keepdim=True) / (heads * real_dim)
+        part = (part / torch.sqrt(ms + eps) * w).reshape(T, heads, D)
+        if cos is not None:
+            rot = 2 * cos.shape[1]
+            c, s = cos[positions.long()].unsqueeze(1), sin[positions.long()].unsqueeze(1)
+            a, b = part[..., 0:rot:2].clone(), part[..., 1:rot:2].clone()
+            part[..., 0:rot:2], part[..., 1:rot:2] = a * c - b * s, b * c + a * s
+        out.append(part.reshape(T, heads * D))
+    return torch.cat(out + [v], dim=1).to(p.dtype)
+
+
 def lanes_step(lanes, count, update=None, read=None, norm_weight=None, eps=0.0, out_dtype=None,
                rows=None, round_parts=False, want=True):
     S = count
@@ -161,7 +217,9 @@ def shift_mix(x, mu, state, seq_of_token, cu, slots, num_seqs):
     return out
 
 
-def tail_update(state, x, channels, rows, cu, slots, num_seqs):
+def tail_update(state, x, channels, rows, cu, slots, num_seqs, bias=None):
+    if bias is not None:
+        x = x[:, :channels] + bias
     for t0, t1, slot in _seqs(cu, slots, num_seqs):
         old = state[slot, :channels * rows].reshape(rows, channels).clone()
         both = torch.cat([old, x[t0:t1, :channels].float()], dim=0)
@@ -171,8 +229,10 @@ def tail_update(state, x, channels, rows, cu, slots, num_seqs):
 def causal_conv(x, taps, state, seq_of_token, cu, slots, num_seqs, unit_channels=0, unit_group=0,
                 scaled_channels=0, scale=1.0, unit_eps=0.0, rest_group=256, bias=None,
                 out_dtype=torch.float32, activation=True, blend=None, blend_from=0,
-                blend_weight=0.0):
+                blend_weight=0.0, in_bias=None):
     C, K = taps.shape
+    if in_bias is not None:
+        x = x[:, :C] + in_bias
     out = torch.empty((x.shape[0], C), dtype=torch.float32)
     for t0, t1, slot in _seqs(cu, slots, num_seqs):
         before = state[slot, :C * (K - 1)].reshape(K - 1, C) if K > 1 else x.new_zeros((0, C))
@@ -361,6 +421,46 @@ def delta_scan(q, k, v, b_raw, a_raw, a_log, dt_bias, state, cu, slots, num_seqs
     return out
 
 
+def channel_delta_scan(q, k, v, b_raw, z, a_log, dt_bias, state, cu, slots, num_seqs, heads,
+                       kv_heads, dk, dv, tiled=None):
+    T = q.shape[0]
+    out = torch.empty((T, heads * dv), dtype=torch.float32)
+    g = torch.nn.functional.softplus(z + dt_bias).reshape(T, heads, dk)
+    g = torch.exp(-torch.exp(a_log).reshape(1, heads, 1) * g)
+    beta = torch.sigmoid(b_raw)
+    for t0, t1, slot in _seqs(cu, slots, num_seqs):
+        S = state[slot, :heads * dv * dk].reshape(heads, dv, dk).clone()     # [head][value][key]
+        for t in range(t0, t1):
+            for h in range(heads):
+                j = h // (heads // kv_heads)
+                kt, qt = k[t, j * dk:(j + 1) * dk], q[t, j * dk:(j + 1) * dk]
+                S[h] = S[h] * g[t, h]
+                u = beta[t, h] * (v[t, h * dv:(h + 1) * dv] - S[h] @ kt)
+                S[h] = S[h] + torch.outer(u, kt)
+                out[t, h * dv:(h + 1) * dv] = S[h] @ qt
+        state[slot, :heads * dv * dk] = S.reshape(-1)
+    return out
+
+
+def rglru_scan(u, gates, r_bias, i_bias, rate, y, y_bias, state, cu, slots, num_seqs, blocks,
+               longest=None):
+    T, C = u.shape
+    parts = gates.reshape(T, blocks, 2, C // blocks)
+    r = torch.sigmoid(parts[:, :, 0].reshape(T, C) + r_bias)
+    i = torch.sigmoid(parts[:, :, 1].reshape(T, C) + i_bias)
+    log_a = rate * r
+    drive = torch.sqrt(-torch.expm1(2.0 * log_a)) * i * u.float()
+    a, gate = torch.exp(log_a), gelu_tanh(y + y_bias)
+    out = torch.empty((T, C), dtype=torch.float32)
+    for t0, t1, slot in _seqs(cu, slots, num_seqs):
+        S = state[slot, :C].clone()
+        for t in range(t0, t1):
+            S = a[t] * S + drive[t]
+            out[t] = S * gate[t]
+        state[slot, :C] = S
+    return out.to(u.dtype)
+
+
 def decay_scan(r, k, v, z, w0, bonus, state, cu, slots, num_seqs, heads, d, tiled=None):
     T = r.shape[0]
     out = torch.empty((T, heads * d), dtype=torch.float32)
@@ -435,15 +535,16 @@ def copy_pages(pages, src, dst):
 
 
 def attention_planner(num_heads, num_kv_heads, head_dim, dtype, biased=False, shaped=False,
-                      plain=False):
+                      plain=False, span=0):
     from rust_llm_inference_server_amd.ops.attention_plan import AttentionPlanner
-    return AttentionPlanner(num_heads, num_kv_heads, head_dim, matrix=dtype == torch.bfloat16)
+    return AttentionPlanner(num_heads, num_kv_heads, head_dim, matrix=dtype == torch.bfloat16,
+                            span=span)
 
 
 def paged_attention(qkv, num_heads, num_kv_heads, head_dim, k_pages, v_pages, page_size,
                     block_tables, step, scale, window=None, force=None, plan=None,
                     bias_slopes=None, counters=None, head_scales=None, softcap=0.0, sinks=None,
-                    keep_first=0):
+                    keep_first=0, chunk=None):
     assert bias_slopes is None, "the test double adds no bias"
     T = qkv.shape[0]
     nh, nkv, d = num_heads, num_kv_heads, head_dim
@@ -455,6 +556,8 @@ def paged_attention(qkv, num_heads, num_kv_heads, head_dim, k_pages, v_pages, pa
     for t in range(T):
         table = block_tables[seq_of[t]].tolist()
         lo = max(0, pos[t] - window + 1) if window else 0
+        if chunk:
+            lo = pos[t] - pos[t] % chunk
         keys = list(range(0, min(keep_first, lo) if window else 0)) + list(range(lo, pos[t] + 1))
         k = torch.stack([k_pages[table[p // page_size], :, p % page_size, :] for p in keys]).float()
         v = torch.stack([v_pages[table[p // page_size], :, :, p % page_size] for p in keys]).float()
@@ -475,13 +578,13 @@ def paged_attention(qkv, num_heads, num_kv_heads, head_dim, k_pages, v_pages, pa
 def rope_attention(qkv, num_heads, num_kv_heads, head_dim, cos, sin, positions, slots, k_pages,
                    v_pages, page_size, block_tables, step, scale, window=None, write_kv=True,
                    plan=None, interleaved=False, bias_slopes=None, counters=None,
-                   head_scales=None, softcap=0.0, sinks=None, keep_first=0):
+                   head_scales=None, softcap=0.0, sinks=None, keep_first=0, chunk=None):
     own = 0 if qkv.shape[1] == num_heads * head_dim else num_kv_heads     # queries alone?
     rope_kv_write(qkv, num_heads, own, head_dim, cos, sin, positions, slots, k_pages,
                   v_pages, page_size, write_kv=write_kv and own > 0)
     return paged_attention(qkv, num_heads, num_kv_heads, head_dim, k_pages, v_pages, page_size,
                            block_tables, step, scale, window, head_scales=head_scales,
-                           softcap=softcap, sinks=sinks, keep_first=keep_first)
+                           softcap=softcap, sinks=sinks, keep_first=keep_first, chunk=chunk)
 
 
 def _lowbias32(x):
@@ -524,6 +627,7 @@ def install(monkeypatch) -> None:
                  "latent_mfma_ok",
                  "sigmoid_gate_", "route", "routed_units", "router_logits", "gelu_tanh",
                  "depth_mix_", "decay_attention", "gelu_erf", "lanes_step", "head_prepare_",
-                 "head_gate_"):
+                 "head_gate_", "geglu", "linear_geglu", "norm_join", "side_gate_", "embed_pairs",
+                 "row_prepare", "channel_delta_scan", "rglru_scan"):
         monkeypatch.setattr(ops, name, globals()[name])
     monkeypatch.setattr(runner, "default_device", lambda: torch.device("cpu"))
