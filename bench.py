@@ -55,7 +55,11 @@ layers alternate between attention over every earlier key with biases, head norm
 every second of them on the keys and values of the one before, and attention with a window of
 1,024 that also keeps the first 64 keys, with a gate per head; feed-forwards alternate between a
 dense GELU unit and a mixture of squared-ReLU units).  ``--design lagedra,pamolix`` puts it
-beside its closest kin."""
+beside its closest kin.
+``--design ralitar`` times the Ralitar design (norms behind the sublayers, a table of token pairs,
+a token input per layer; of every four layers two are the delta rule with a decay per key channel,
+one is a gated linear recurrence and one attention inside chunks of 1,024); its closest kin is
+Gipotar: ``--design gipotar,ralitar``."""
 import argparse
 import copy
 import json
@@ -313,6 +317,32 @@ def pamolix_like(cfg: dict) -> dict:
             "embedding": {"scale": 1.0}, "norm": {"eps": 1e-6}, "streams": 2, "layers": layers}
 
 
+def ralitar_like(cfg: dict) -> dict:
+    """A Ralitar configuration at the sizes of a Llama preset: the same width, depth,
+    feed-forward width, vocabulary and attention heads; of every four layers two are the delta
+    rule (heads of 128, half as many q/k heads, low-rank pairs of rank 128), one is a gated linear
+    recurrence as wide as the model (eight blocks of gates) and one attention inside chunks of
+    1,024 (half of every head rotated, stretched by 4, cap 30), each with a feed-forward; a token
+    input of 128 numbers per layer and a pair table of 200,003 rows."""
+    W, d = cfg["hidden_size"], cfg["head_dim"]
+    mlp = {"kind": "dense", "ff": cfg["intermediate_size"]}
+    heads = max(1, W // 128)
+    delta = {"type": "channel_delta", "mlp": mlp, "mixer": {
+        "heads": heads, "kv_heads": max(1, heads // 2), "dim": 128, "vdim": 128, "conv": 4,
+        "decay_rank": 128, "gate_rank": 128}}
+    rglru = {"type": "rglru", "mlp": mlp, "mixer": {"width": W, "blocks": 8, "conv": 4}}
+    attention = {"type": "attention", "mlp": mlp, "mixer": {
+        "heads": cfg["num_attention_heads"], "kv_heads": cfg["num_key_value_heads"], "dim": d,
+        "vdim": d, "scale": d ** -0.5, "mask": {"size": 1024}, "softcap": 30.0,
+        "rot": {"dims": d // 2, "base": cfg["rope_theta"],
+                "scaling": {"factor": 4.0, "low": 1.0, "high": 4.0, "original": 8192}}}}
+    order = (delta, rglru, delta, attention)
+    return {"architecture": "Ralitar", "vocab": cfg["vocab_size"], "width": W,
+            "embedding": {"bigram": {"buckets": 200003, "mul_prev": 1000003, "mul_cur": 31}},
+            "token_side": {"dim": 128}, "norm": {"eps": 1e-5},
+            "layers": [copy.deepcopy(order[i % 4]) for i in range(cfg["num_hidden_layers"])]}
+
+
 def step_bytes_of(model, batch: int, mean_context: float) -> float:
     """What a decode step of any model has to move: every tensor its parts hold once (the
     embedding table only where the head shares it), each live request's cached positions, and
@@ -325,6 +355,10 @@ def step_bytes_of(model, batch: int, mean_context: float) -> float:
     table = model.embedding.weight
     if model.head.weight.data_ptr() != table.data_ptr():
         total -= table.numel() * table.element_size()
+    # tables of which a step reads a row per token
+    tables = [getattr(model.embedding, "bigram", None)] + [
+        getattr(getattr(layer, "side", None), "table", None) for layer in model.layers[:1]]
+    total -= sum(t.numel() * t.element_size() for t in tables if t is not None)
     total -= routed_idle_bytes(model, batch)
     per_position = 0.0                    # every run reads its group's pages, its own or not
     for b in model.bindings:
@@ -421,7 +455,7 @@ def compare_designs(args) -> int:
         longest = max(T, args.points_context + new + warm + 16) + 64
         base["max_position_embeddings"] = min(base["max_position_embeddings"], longest)
         like = {"gipotar": gipotar_like, "bekunex": bekunex_like, "lagedra": lagedra_like,
-                "pamolix": pamolix_like}
+                "pamolix": pamolix_like, "ralitar": ralitar_like}
         for design, cfg in [("llama", base)] + [(d, like[d](base)) for d in args.design.split(",")]:
             vocab = base["vocab_size"]
             model = random_model(cfg, seed=0, dtype=args.dtype, max_positions=longest)
@@ -483,7 +517,7 @@ def main() -> int:
                     help="time the Gipotar design beside the Llama presets of --sizes instead")
     ap.add_argument("--design", default="gipotar",
                     help="the designs that --designs times beside Llama, with commas between "
-                         "them: gipotar, bekunex, lagedra")
+                         "them: gipotar, bekunex, lagedra, pamolix, ralitar")
     ap.add_argument("--sizes", default="llama-3.2-1b,llama-3.2-3b",
                     help="presets whose sizes the two designs of --designs are built at")
     args = ap.parse_args()

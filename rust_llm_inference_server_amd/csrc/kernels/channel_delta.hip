@@ -10,6 +10,7 @@
 // channel] in the request's slot, a wave owns a few value channels of one (sequence, head), lane i
 // holds S[i][j] (and i + 64, ... for more than 64 key channels).
 #include "scan.h"
+#include "tile_mma.h"
 
 namespace {
 
@@ -299,7 +300,445 @@ __global__ __launch_bounds__(256) void channel_delta_tiled_kernel(const ChannelD
     }
 }
 
+// ------------------------------------------------------------------------ long portions
+// Chunks of kChunk tokens on the matrix cores, float32 products (v_mfma_f32_16x16x4_f32).  With S0
+// the state in front of a chunk and G(t, s) the products of the decays of tokens s + 1 .. t per
+// key channel (G(t) from the chunk's start), the writes u_t of a chunk solve
+//   u_t = beta_t (v_t - S0^T (G(t) k_t) - sum_{s<t} A[t][s] u_s),  A[t][s] = sum_i G(t,s) k_t k_s,
+// a unit lower triangular system that does not depend on S0: with U0 its solution for the right
+// hand side beta v and W that for beta (G k),  U = U0 - W S0, and
+//   o_t = S0^T (G(t) q_t) + sum_{s<=t} B[t][s] u_s,          B[t][s] = sum_i G(t,s) q_t k_s,
+//   S  <- G(n) S0 + sum_s (G(n, s) k_s) u_s^T.
+// Three launches: what does not depend on the state, chunk by chunk and head by head side by
+// side; the states, chunk after chunk, a workgroup per 16 value channels; the read-outs, side by
+// side again.
+//
+// No decay is ever divided by: inside 16 tokens G(t, s) is formed by multiplying the decays up from s;
+// between blocks of 16 it is split at the later block's start into two factors that are at most
+// one, the exponentials of sums of logarithms that all have one sign.  So strong decays
+// underflow to zero and nothing overflows or cancels.
+constexpr int kChunk = 64, kSub = 16, kSubs = kChunk / kSub;
+
+struct ChannelDeltaChunks {
+  ChannelDeltaArgs a;
+  int num_seqs, max_chunks, dvp;   // dvp: value channels rounded up to 16
+  float *w, *qt, *kt, *u, *b, *gc, *s0;
+};
+
+// Per (chunk, head): w (64, DK), qt (64, DK) = G q, kt (DK, 64) = G(n, s) k, u (dvp, 64), b (64, 64),
+// gc (DK) = G(n), s0 (dvp, DK).
+template <int DK>
+__host__ __device__ constexpr long long chunk_floats(int dvp) {
+  return 3LL * kChunk * DK + (long long)dvp * kChunk + kChunk * kChunk + DK + (long long)dvp * DK;
+}
+
+template <int DK>
+struct PrepLds {
+  static constexpr int kStride = DK + 4;
+  float k[kChunk][kStride], q[kChunk][kStride], g[kChunk][kStride], p[kChunk][kStride];
+  float a[kChunk][kChunk + 4];
+  float end[kSubs][DK];
+  float beta[kChunk];
+};
+
+__device__ __forceinline__ float4 ld4(const float* p) { return *(const float4*)p; }
+__device__ __forceinline__ void mfma4(const float4& a, const float4& b, mma_f32x4& acc) {
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.x, b.x, acc, 0, 0, 0);
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.y, b.y, acc, 0, 0, 0);
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.z, b.z, acc, 0, 0, 0);
+  acc = __builtin_amdgcn_mfma_f32_16x16x4f32(a.w, b.w, acc, 0, 0, 0);
+}
+
+template <int DK>
+__global__ __launch_bounds__(256) void channel_delta_prepare_kernel(const ChannelDeltaChunks c) {
+  extern __shared__ __attribute__((aligned(16))) char prep_smem[];
+  PrepLds<DK>& L = *reinterpret_cast<PrepLds<DK>*>(prep_smem);
+  const ChannelDeltaArgs& a = c.a;
+  const int chunk = blockIdx.x, head = blockIdx.y;
+  int t0, t1;
+  if (!chunk_span(a.cu, c.num_seqs, kChunk, chunk, t0, t1)) return;   // (the whole workgroup)
+  const int n = t1 - t0;
+  const int tid = threadIdx.x, lane = tid % kWave, wave = tid / kWave;
+  const int kh = head / (a.heads / a.kv_heads);
+  const int dk = a.dk, dv = a.dv;
+  const long long at = (long long)chunk * a.heads + head;
+  float* ws_w = c.w + at * kChunk * DK;
+  float* ws_qt = c.qt + at * kChunk * DK;
+  float* ws_kt = c.kt + at * kChunk * DK;
+  float* ws_u = c.u + at * c.dvp * kChunk;
+  float* ws_b = c.b + at * kChunk * kChunk;
+  const float neg_a = -expf(a.a_log[head]);
+  if (tid < kChunk) {
+    const float raw = a.b_raw[(long long)(t0 + min(tid, n - 1)) * a.ldb + head];
+    L.beta[tid] = tid < n ? sigmoidf_(raw) : 0.f;
+  }
+  // A thread owns (channel, block of 16 tokens) items: their inputs, the logarithms of the decays
+  // (kept in registers), the running sums from the block's start.  Tokens past the end carry zero
+  // keys and no decay.
+  constexpr int ITEMS = DK * kSubs / 256;
+  float lg[ITEMS][kSub];
+#pragma unroll
+  for (int it = 0; it < ITEMS; ++it) {
+    const int id = tid + it * 256, ch = id % DK, sub = id / DK;
+    const int ic = min(ch, dk - 1);
+    const float bias = a.dt_bias[head * dk + ic];
+    float kv[kSub], qv[kSub];
+#pragma unroll
+    for (int j = 0; j < kSub; ++j) {
+      const long long t = t0 + min(sub * kSub + j, n - 1);
+      lg[it][j] = a.z[t * a.ldz + head * dk + ic];
+      kv[j] = a.k[t * a.ldqkv + kh * dk + ic];
+      qv[j] = a.q[t * a.ldqkv + kh * dk + ic];
+    }
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < kSub; ++j) {
+      const int t = sub * kSub + j;
+      const bool live = t < n && ch < dk;
+      lg[it][j] = live ? neg_a * softplusf_(lg[it][j] + bias) : 0.f;
+      sum += lg[it][j];
+      L.k[t][ch] = live ? kv[j] : 0.f;
+      L.q[t][ch] = live ? qv[j] : 0.f;
+      L.g[t][ch] = expf(lg[it][j]);
+      L.p[t][ch] = sum;
+    }
+    L.end[sub][ch] = sum;
+  }
+  __syncthreads();
+  // Blocks of 16 x 16 on the diagonal: lane l carries column s = l % 16 for a quarter of the
+  // channels; w = G(t, s) k_s is multiplied up as t goes on.  (For t <= s the entries of A mean
+  // nothing and are not read; those of B are zero for t < s.)
+  {
+    const int s = lane % 16, gq = lane / 16, r0 = wave * kSub;
+    float acc_a[kSub], acc_b[kSub];
+#pragma unroll
+    for (int j = 0; j < kSub; ++j) acc_a[j] = acc_b[j] = 0.f;
+    for (int m = 0; m < DK / 16; ++m) {
+      const int i = 16 * m + 4 * gq;
+      const float4 ks = ld4(&L.k[r0 + s][i]);
+      float4 w = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll
+      for (int j = 0; j < kSub; ++j) {
+        const float4 g4 = ld4(&L.g[r0 + j][i]), k4 = ld4(&L.k[r0 + j][i]), q4 = ld4(&L.q[r0 + j][i]);
+        const bool own = j == s;
+        w.x = own ? ks.x : w.x * g4.x;
+        w.y = own ? ks.y : w.y * g4.y;
+        w.z = own ? ks.z : w.z * g4.z;
+        w.w = own ? ks.w : w.w * g4.w;
+        acc_a[j] += (k4.x * w.x + k4.y * w.y) + (k4.z * w.z + k4.w * w.w);
+        acc_b[j] += (q4.x * w.x + q4.y * w.y) + (q4.z * w.z + q4.w * w.w);
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < kSub; ++j) {
+      acc_a[j] = xor32_sum(xor16_sum(acc_a[j]));
+      acc_b[j] = xor32_sum(xor16_sum(acc_b[j]));
+      if (j / 4 == gq) {
+        L.a[r0 + j][r0 + s] = acc_a[j];
+        ws_b[(r0 + j) * kChunk + r0 + s] = acc_b[j];
+      }
+    }
+  }
+  __syncthreads();
+  // The decays make room for the sums of the logarithms behind a token, up to its block's end; on
+  // the way, what the state's update and the read-out take: G(n, s) k and G q.
+#pragma unroll
+  for (int it = 0; it < ITEMS; ++it) {
+    const int id = tid + it * 256, ch = id % DK, sub = id / DK;
+    float before = 0.f, behind = 0.f;
+    for (int r = 0; r < sub; ++r) before += L.end[r][ch];
+    for (int r = sub + 1; r < kSubs; ++r) behind += L.end[r][ch];
+    float suffix = 0.f, khat[kSub];
+#pragma unroll
+    for (int j = kSub - 1; j >= 0; --j) {
+      const int t = sub * kSub + j;
+      L.g[t][ch] = suffix;
+      khat[j] = L.k[t][ch] * expf(suffix + behind);
+      suffix += lg[it][j];
+      ws_qt[t * DK + ch] = L.q[t][ch] * expf(before + L.p[t][ch]);
+    }
+#pragma unroll
+    for (int j = 0; j < kSub; j += 4)
+      *(float4*)(ws_kt + ch * kChunk + sub * kSub + j) =
+          make_float4(khat[j], khat[j + 1], khat[j + 2], khat[j + 3]);
+    if (sub == kSubs - 1) c.gc[at * DK + ch] = expf(before + L.end[sub][ch]);
+  }
+  __syncthreads();
+  // Blocks below the diagonal: block ba against an earlier block bb, G(t, s) split at ba's start.
+  for (int pair = wave; pair < kSubs * (kSubs - 1) / 2; pair += 4) {
+    const int ba = pair < 1 ? 1 : (pair < 3 ? 2 : 3), bb = pair - ba * (ba - 1) / 2;
+    const int row = ba * kSub + lane % 16, col = bb * kSub + lane % 16, g = lane / 16;
+    mma_f32x4 acc_a = {0.f, 0.f, 0.f, 0.f}, acc_b = {0.f, 0.f, 0.f, 0.f};
+    for (int m = 0; m < DK / 16; ++m) {
+      const int i = 16 * m + 4 * g;
+      float4 between = ld4(&L.g[col][i]);
+      for (int r = bb + 1; r < ba; ++r) {
+        const float4 e = ld4(&L.end[r][i]);
+        between.x += e.x;
+        between.y += e.y;
+        between.z += e.z;
+        between.w += e.w;
+      }
+      const float4 p = ld4(&L.p[row][i]);
+      float4 kr = ld4(&L.k[row][i]), qr = ld4(&L.q[row][i]), kc = ld4(&L.k[col][i]);
+      const float4 e = make_float4(expf(p.x), expf(p.y), expf(p.z), expf(p.w));
+      kr.x *= e.x; kr.y *= e.y; kr.z *= e.z; kr.w *= e.w;
+      qr.x *= e.x; qr.y *= e.y; qr.z *= e.z; qr.w *= e.w;
+      kc.x *= expf(between.x); kc.y *= expf(between.y);
+      kc.z *= expf(between.z); kc.w *= expf(between.w);
+      mfma4(kr, kc, acc_a);
+      mfma4(qr, kc, acc_b);
+    }
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = ba * kSub + 4 * g + i;
+      L.a[t][col] = acc_a[i];
+      ws_b[t * kChunk + col] = acc_b[i];
+    }
+  }
+  __syncthreads();
+  // The triangular system, a thread per column: key channels (W) first, value channels (U0) behind.
+  for (int col = tid; col < DK + c.dvp; col += 256) {
+    float x[kChunk];
+    if (col < DK) {
+#pragma unroll
+      for (int sub = 0; sub < kSubs; ++sub) {
+        float before = 0.f;
+        for (int r = 0; r < sub; ++r) before += L.end[r][col];
+#pragma unroll
+        for (int j = 0; j < kSub; ++j) {
+          const int t = sub * kSub + j;
+          x[t] = L.k[t][col] * expf(before + L.p[t][col]);
+        }
+      }
+    } else {
+      const float* v = a.v + (long long)t0 * a.ldqkv + head * dv + min(col - DK, dv - 1);
+#pragma unroll
+      for (int t = 0; t < kChunk; ++t) x[t] = v[(long long)min(t, n - 1) * a.ldqkv];
+      const bool real = col - DK < dv;
+#pragma unroll
+      for (int t = 0; t < kChunk; ++t) x[t] = (real && t < n) ? x[t] : 0.f;
+    }
+#pragma unroll
+    for (int t = 0; t < kChunk; ++t) {
+      float s4[4] = {x[t], 0.f, 0.f, 0.f};
+#pragma unroll
+      for (int s = 0; s < t; s += 4) {
+        const float4 r = ld4(&L.a[t][s]);
+        s4[0] -= r.x * x[s];
+        if (s + 1 < t) s4[1] -= r.y * x[s + 1];
+        if (s + 2 < t) s4[2] -= r.z * x[s + 2];
+        if (s + 3 < t) s4[3] -= r.w * x[s + 3];
+      }
+      x[t] = L.beta[t] * ((s4[0] + s4[1]) + (s4[2] + s4[3]));
+    }
+    if (col < DK) {
+#pragma unroll
+      for (int t = 0; t < kChunk; ++t) ws_w[t * DK + col] = x[t];
+    } else {
+#pragma unroll
+      for (int t = 0; t < kChunk; t += 4)
+        *(float4*)(ws_u + (long long)(col - DK) * kChunk + t) = make_float4(x[t], x[t + 1], x[t + 2], x[t + 3]);
+    }
+  }
+}
+
+// The states: a workgroup per (16 value channels, head, sequence) walks the sequence's chunks.  Wave
+// w owns the key channels of its DK / 64 tiles of 16 (registers: rows 4 (lane / 16) + i, column
+// lane % 16) and 16 tokens of U.  A chunk's operands are asked for one chunk ahead.
+template <int DK>
+__global__ __launch_bounds__(256) void channel_delta_states_kernel(const ChannelDeltaChunks c) {
+  constexpr int KT = DK / 64, KM = DK / 16, TM = kChunk / 16;
+  __shared__ __attribute__((aligned(16))) float ssm[16][DK + 4], usm[16][kChunk + 4];
+  const ChannelDeltaArgs& a = c.a;
+  const int head = blockIdx.y, s = blockIdx.z;
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int l16 = lane % 16, g = lane / 16;
+  const int col = blockIdx.x * 16 + l16;
+  const int dk = a.dk, dv = a.dv;
+  const int first = chunks_before(a.cu, s, kChunk);
+  const int chunks = (a.cu[s + 1] - a.cu[s] + kChunk - 1) / kChunk;
+  if (chunks == 0) return;
+  float* base = a.state + (long long)a.slots[s] * a.state_stride + (long long)head * dv * dk;
+  mma_f32x4 S[KT];
+#pragma unroll
+  for (int j = 0; j < KT; ++j) {
+    const int key = (wave * KT + j) * 16 + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const bool live = key + i < dk && col < dv;
+      const float v = base[live ? (long long)col * dk + key + i : 0];
+      S[j][i] = live ? v : 0.f;
+    }
+    *(float4*)&ssm[l16][key] = make_float4(S[j][0], S[j][1], S[j][2], S[j][3]);
+  }
+  float4 wf[KM], kf[KT][TM], uf, gf[KT];
+  auto ask = [&](int chunk) {
+    const long long at = (long long)(first + chunk) * a.heads + head;
+    const float* w = c.w + at * kChunk * DK + (wave * 16 + l16) * DK + 4 * g;
+#pragma unroll
+    for (int m = 0; m < KM; ++m) wf[m] = ld4(w + 16 * m);
+    uf = ld4(c.u + (at * c.dvp + col) * kChunk + wave * 16 + 4 * g);
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+      const int tile = (wave * KT + j) * 16;
+      const float* kt = c.kt + at * kChunk * DK + (tile + l16) * kChunk + 4 * g;
+#pragma unroll
+      for (int m = 0; m < TM; ++m) kf[j][m] = ld4(kt + 16 * m);
+      gf[j] = ld4(c.gc + at * DK + tile + 4 * g);
+    }
+  };
+  ask(0);
+  __syncthreads();
+  for (int k = 0; k < chunks; ++k) {
+    const long long at = (long long)(first + k) * a.heads + head;
+    float* s0 = c.s0 + (at * c.dvp + col) * DK;
+#pragma unroll
+    for (int j = 0; j < KT; ++j)
+      *(float4*)(s0 + (wave * KT + j) * 16 + 4 * g) = make_float4(S[j][0], S[j][1], S[j][2], S[j][3]);
+    mma_f32x4 acc = {0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+    for (int m = 0; m < KM; ++m) mfma4(wf[m], ld4(&ssm[l16][16 * m + 4 * g]), acc);
+    const float4 u = make_float4(uf.x - acc[0], uf.y - acc[1], uf.z - acc[2], uf.w - acc[3]);
+    *(float4*)&usm[l16][wave * 16 + 4 * g] = u;
+    *(float4*)(c.u + (at * c.dvp + col) * kChunk + wave * 16 + 4 * g) = u;
+    float4 kn[KT][TM];
+#pragma unroll
+    for (int j = 0; j < KT; ++j) {
+#pragma unroll
+      for (int m = 0; m < TM; ++m) kn[j][m] = kf[j][m];
+      S[j][0] *= gf[j].x;
+      S[j][1] *= gf[j].y;
+      S[j][2] *= gf[j].z;
+      S[j][3] *= gf[j].w;
+    }
+    ask(k + 1 < chunks ? k + 1 : k);          // (the last chunk's again: not used)
+    __syncthreads();
+#pragma unroll
+    for (int m = 0; m < TM; ++m) {
+      const float4 ub = ld4(&usm[l16][16 * m + 4 * g]);
+#pragma unroll
+      for (int j = 0; j < KT; ++j) mfma4(kn[j][m], ub, S[j]);
+    }
+#pragma unroll
+    for (int j = 0; j < KT; ++j)
+      *(float4*)&ssm[l16][(wave * KT + j) * 16 + 4 * g] = make_float4(S[j][0], S[j][1], S[j][2], S[j][3]);
+    __syncthreads();
+  }
+#pragma unroll
+  for (int j = 0; j < KT; ++j) {
+    const int key = (wave * KT + j) * 16 + 4 * g;
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+      if (key + i < dk && col < dv) base[(long long)col * dk + key + i] = S[j][i];
+  }
+}
+
+// The read-outs: wave w takes 16 tokens of a chunk against up to 64 value channels.
+template <int DK>
+__global__ __launch_bounds__(256) void channel_delta_outputs_kernel(const ChannelDeltaChunks c) {
+  constexpr int NB = 4;
+  const ChannelDeltaArgs& a = c.a;
+  const int chunk = blockIdx.x, head = blockIdx.y, c0 = blockIdx.z * 16 * NB;
+  int t0, t1;
+  if (!chunk_span(a.cu, c.num_seqs, kChunk, chunk, t0, t1)) return;
+  const int lane = threadIdx.x % kWave, wave = threadIdx.x / kWave;
+  const int l16 = lane % 16, g = lane / 16;
+  if (t0 + wave * 16 >= t1) return;
+  const long long at = (long long)chunk * a.heads + head;
+  const float* q = c.qt + at * kChunk * DK + (wave * 16 + l16) * DK + 4 * g;
+  const float* b = c.b + at * kChunk * kChunk + (wave * 16 + l16) * kChunk + 4 * g;
+  const float *s[NB], *u[NB];
+  mma_f32x4 acc[NB];
+#pragma unroll
+  for (int x = 0; x < NB; ++x) {
+    const int col = min(c0 + x * 16, c.dvp - 16) + l16;      // (past the end: not stored)
+    s[x] = c.s0 + (at * c.dvp + col) * DK + 4 * g;
+    u[x] = c.u + (at * c.dvp + col) * kChunk + 4 * g;
+    acc[x] = mma_f32x4{0.f, 0.f, 0.f, 0.f};
+  }
+#pragma unroll 4
+  for (int m = 0; m < DK / 16; ++m) {
+    const float4 qa = ld4(q + 16 * m);
+#pragma unroll
+    for (int x = 0; x < NB; ++x) mfma4(qa, ld4(s[x] + 16 * m), acc[x]);
+  }
+  for (int m = 0; m <= wave; ++m) {
+    const float4 ba = ld4(b + 16 * m);
+#pragma unroll
+    for (int x = 0; x < NB; ++x) mfma4(ba, ld4(u[x] + 16 * m), acc[x]);
+  }
+#pragma unroll
+  for (int x = 0; x < NB; ++x) {
+    const int col = c0 + x * 16 + l16;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+      const int t = t0 + wave * 16 + 4 * g + i;
+      if (t < t1 && col < a.dv) a.out[(long long)t * a.ldo + head * a.dv + col] = acc[x][i];
+    }
+  }
+}
+
+template <int DK>
+int launch_channel_delta_chunks(ChannelDeltaChunks c, float* ws, hipStream_t stream) {
+  const long long n = (long long)c.max_chunks * c.a.heads;
+  c.w = ws;
+  c.qt = c.w + n * kChunk * DK;
+  c.kt = c.qt + n * kChunk * DK;
+  c.u = c.kt + n * kChunk * DK;
+  c.b = c.u + n * c.dvp * kChunk;
+  c.gc = c.b + n * kChunk * kChunk;
+  c.s0 = c.gc + n * DK;
+  static LdsGrant grant;
+  constexpr int bytes = (int)sizeof(PrepLds<DK>);
+  static_assert(bytes <= 160 * 1024, "the chunk does not fit the LDS");
+  const hipError_t e = grant_lds(grant, (const void*)&channel_delta_prepare_kernel<DK>, bytes);
+  RLIS_REQUIRE(e == hipSuccess, "channel_delta_chunks: %d bytes of LDS: %s", bytes, hipGetErrorString(e));
+  channel_delta_prepare_kernel<DK><<<dim3(c.max_chunks, c.a.heads), 256, bytes, stream>>>(c);
+  RLIS_LAUNCH_CHECK("channel_delta_chunks");
+  channel_delta_states_kernel<DK><<<dim3(c.dvp / 16, c.a.heads, c.num_seqs), 256, 0, stream>>>(c);
+  RLIS_LAUNCH_CHECK("channel_delta_chunks");
+  channel_delta_outputs_kernel<DK><<<dim3(c.max_chunks, c.a.heads, ceil_div(c.dvp, 64)), 256, 0, stream>>>(c);
+  RLIS_LAUNCH_CHECK("channel_delta_chunks");
+  return 0;
+}
+
 }  // namespace
+
+// Floats of workspace per (chunk, head) that rlis_channel_delta_chunks needs.
+RLIS_API long long rlis_channel_delta_chunk_floats(int dk, int dv) {
+  const int dvp = ceil_div(dv, 16) * 16;
+  return dk <= 64 ? chunk_floats<64>(dvp) : chunk_floats<128>(dvp);
+}
+
+// rlis_channel_delta_scan for steps with long portions; max_chunks: at least the chunks of 64
+// tokens of all sequences together; ws: max_chunks * heads * rlis_channel_delta_chunk_floats floats,
+// 16-byte aligned.
+RLIS_API int rlis_channel_delta_chunks(float* out, long long ldo, const float* q, const float* k,
+                                       const float* v, long long ldqkv, const float* b_raw,
+                                       long long ldb, const float* z, long long ldz,
+                                       const float* a_log, const float* dt_bias, float* state,
+                                       long long state_stride, const int* cu, const int* slots,
+                                       int num_seqs, int heads, int kv_heads, int dk, int dv,
+                                       int max_chunks, float* ws, hipStream_t stream) {
+  RLIS_REQUIRE(heads > 0 && kv_heads > 0 && heads % kv_heads == 0 && dk > 0 && dv > 0,
+               "channel_delta_chunks: bad sizes heads=%d kv_heads=%d dk=%d dv=%d", heads, kv_heads, dk, dv);
+  RLIS_REQUIRE(dk <= 128, "channel_delta_chunks: %d key channels, at most 128", dk);
+  RLIS_REQUIRE(state_stride >= (long long)heads * dk * dv, "channel_delta_chunks: the state is too short");
+  RLIS_REQUIRE(ldz >= (long long)heads * dk && ldb >= heads && ldo >= (long long)heads * dv,
+               "channel_delta_chunks: rows shorter than the heads they hold");
+  RLIS_REQUIRE(heads <= 65535 && num_seqs <= 65535 && max_chunks > 0 && ws && (uintptr_t)ws % 16 == 0,
+               "channel_delta_chunks: %d chunks, or no aligned workspace", max_chunks);
+  if (num_seqs <= 0) return 0;
+  ChannelDeltaChunks c;
+  c.a = ChannelDeltaArgs{out, ldo, q, k, v, ldqkv, b_raw, ldb, z, ldz, a_log, dt_bias, state,
+                         state_stride, cu, slots, heads, kv_heads, dk, dv};
+  c.num_seqs = num_seqs;
+  c.max_chunks = max_chunks;
+  c.dvp = ceil_div(dv, 16) * 16;
+  return dk <= 64 ? launch_channel_delta_chunks<64>(c, ws, stream)
+                  : launch_channel_delta_chunks<128>(c, ws, stream);
+}
 
 RLIS_API int rlis_channel_delta_scan(float* out, long long ldo, const float* q, const float* k,
                                      const float* v, long long ldqkv, const float* b_raw,

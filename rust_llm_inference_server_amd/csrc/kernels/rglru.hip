@@ -85,29 +85,12 @@ __global__ __launch_bounds__(256) void rglru_scan_kernel(const RglruArgs a) {
   *slot = rglru_walk<TX, true>(a, c, a.cu[s], a.cu[s + 1], *slot, unused);
 }
 
-// Chunks of all sequences in order; the `index`-th one's sequence and first token (false: there
-// are fewer).
-__device__ __forceinline__ bool rglru_chunk(const RglruArgs& a, int index, int& t0, int& t1) {
-  int left = index;
-  for (int s = 0; s < a.num_seqs; ++s) {
-    const int b = a.cu[s], e = a.cu[s + 1];
-    const int chunks = (e - b + a.chunk - 1) / a.chunk;
-    if (left < chunks) {
-      t0 = b + left * a.chunk;
-      t1 = min(e, t0 + a.chunk);
-      return true;
-    }
-    left -= chunks;
-  }
-  return false;
-}
-
 template <typename TX, bool OUT>
 __global__ __launch_bounds__(256) void rglru_chunk_kernel(const RglruArgs a) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   const int chunk = blockIdx.y;
   int t0, t1;
-  if (c >= a.C || !rglru_chunk(a, chunk, t0, t1)) return;
+  if (c >= a.C || !chunk_span(a.cu, a.num_seqs, a.chunk, chunk, t0, t1)) return;
   float* decay_at = a.ws + (long long)chunk * a.C + c;
   float* sum_at = decay_at + (long long)a.max_chunks * a.C;
   float decay = 1.f;
@@ -125,8 +108,7 @@ __global__ __launch_bounds__(256) void rglru_join_kernel(const RglruArgs a) {
   const int c = blockIdx.x * blockDim.x + threadIdx.x;
   const int s = blockIdx.y;
   if (c >= a.C) return;
-  int first = 0;
-  for (int r = 0; r < s; ++r) first += (a.cu[r + 1] - a.cu[r] + a.chunk - 1) / a.chunk;
+  const int first = chunks_before(a.cu, s, a.chunk);
   const int chunks = (a.cu[s + 1] - a.cu[s] + a.chunk - 1) / a.chunk;
   float* slot = a.state + (long long)a.slots[s] * a.state_stride + c;
   float S = *slot;

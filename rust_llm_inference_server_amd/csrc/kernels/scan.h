@@ -80,3 +80,27 @@ static inline int scan_compute_units() {
   }
   return units;
 }
+
+// Forms that cut every sequence's tokens of the step into chunks of `len` number the chunks of all
+// sequences in order.  The `index`-th chunk's tokens [t0, t1) (false: there are fewer), and the
+// number of chunks in front of a sequence.
+__device__ __forceinline__ bool chunk_span(const int* cu, int num_seqs, int len, int index, int& t0,
+                                           int& t1) {
+  int left = index;
+  for (int s = 0; s < num_seqs; ++s) {
+    const int b = cu[s], e = cu[s + 1];
+    const int chunks = (e - b + len - 1) / len;
+    if (left < chunks) {
+      t0 = b + left * len;
+      t1 = min(e, t0 + len);
+      return true;
+    }
+    left -= chunks;
+  }
+  return false;
+}
+__device__ __forceinline__ int chunks_before(const int* cu, int seq, int len) {
+  int n = 0;
+  for (int s = 0; s < seq; ++s) n += (cu[s + 1] - cu[s] + len - 1) / len;
+  return n;
+}

@@ -35,6 +35,7 @@ _SIGNATURES = {
     "rlis_embed_pairs": [P, P, P, I, P, I, I, I, F, L, L, P, L, P, P, P, P],
     "rlis_row_prepare": [P, P, I, L, I, I, I, I, I, P, P, P, F, P, P, I, P, I, P],
     "rlis_channel_delta_scan": [P, L, P, P, P, L, P, L, P, L, P, P, P, L, P, P, I, I, I, I, I, I, P],
+    "rlis_channel_delta_chunks": [P, L, P, P, P, L, P, L, P, L, P, P, P, L, P, P, I, I, I, I, I, I, P, P],
     "rlis_rglru_scan": [P, I, P, L, P, L, P, P, P, P, L, P, P, L, P, P, I, I, I, I, I, P, P],
     "rlis_clamped_glu": [P, P, I, I, I, F, F, P],
     "rlis_weighted_sum": [P, P, I, F, I, P, I, F, I, L, I, P],
@@ -119,6 +120,8 @@ def load() -> ctypes.CDLL:
     lib.rlis_gemm_bf16_stream_join_tiles.argtypes = [I, I]
     lib.rlis_attn_register_unit.restype = c_int
     lib.rlis_attn_register_unit.argtypes = [I, P, P]
+    lib.rlis_channel_delta_chunk_floats.restype = L
+    lib.rlis_channel_delta_chunk_floats.argtypes = [I, I]
     lib.rlis_norm_linear_max_k.restype = c_int
     lib.rlis_norm_linear_max_k.argtypes = []
     lib.rlis_lt_tune.restype = c_int

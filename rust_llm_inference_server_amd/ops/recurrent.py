@@ -240,15 +240,28 @@ def head_norm_gate(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, he
     return out
 
 
+# A step in which some sequence brings at least CHANNEL_DELTA_CHUNKED_MIN_LONGEST tokens takes the
+# chunked form of the channel-wise delta rule (chunks of CHANNEL_DELTA_CHUNK_LEN tokens on the matrix
+# cores; heads of at most CHANNEL_DELTA_CHUNKED_MAX_DIM key channels), if its workspace stays
+# within CHANNEL_DELTA_CHUNKED_MAX_BYTES.
+CHANNEL_DELTA_CHUNK_LEN = 64
+CHANNEL_DELTA_CHUNKED_MIN_LONGEST = 48
+CHANNEL_DELTA_CHUNKED_MAX_DIM = 128
+CHANNEL_DELTA_CHUNKED_MAX_BYTES = 8 << 30
+
+
 def channel_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b_raw: torch.Tensor,
                        z: torch.Tensor, a_log: torch.Tensor, dt_bias: torch.Tensor,
                        state: torch.Tensor, cu: torch.Tensor, slots: torch.Tensor, num_seqs: int,
-                       heads: int, kv_heads: int, dk: int, dv: int, tiled=None) -> torch.Tensor:
+                       heads: int, kv_heads: int, dk: int, dv: int, tiled=None,
+                       longest: Optional[int] = None) -> torch.Tensor:
     """``delta_scan`` with one decay per head and key channel: per token and head
     ``S <- diag(g) S; u = beta (v - S^T k); S <- S + k u^T; o = S^T q`` with
     ``g[i] = exp(-exp(a_log[head]) * softplus(z[head * dk + i] + dt_bias[head * dk + i]))`` and
     ``beta = sigmoid(b_raw)``.  ``z (T, heads * dk)``, ``b_raw (T, heads)`` float32 with rows of
-    their own strides; everything else as for ``delta_scan``."""
+    their own strides; everything else as for ``delta_scan``.  Steps with long portions
+    (``longest``: the most tokens a sequence brings, None: not known) take the chunked form
+    (``tiled="chunked"``: always); the three forms agree to rounding."""
     ld = _rows(q, "channel_delta_scan q", torch.float32)
     if _rows(k, "channel_delta_scan k", torch.float32) != ld \
             or _rows(v, "channel_delta_scan v", torch.float32) != ld:
@@ -261,6 +274,23 @@ def channel_delta_scan(q: torch.Tensor, k: torch.Tensor, v: torch.Tensor, b_raw:
         raise KernelError("channel_delta_scan: operand shapes do not match the head counts and sizes")
     stride = _state(state, heads * dv * dk, "channel_delta_scan")
     out = torch.empty((T, heads * dv), dtype=torch.float32, device=q.device)
+    chunked = tiled == "chunked"
+    max_chunks = T // CHANNEL_DELTA_CHUNK_LEN + num_seqs            # an upper bound, known on the host
+    if tiled is None and longest is not None and dk <= CHANNEL_DELTA_CHUNKED_MAX_DIM \
+            and longest >= CHANNEL_DELTA_CHUNKED_MIN_LONGEST:
+        per = lib.load().rlis_channel_delta_chunk_floats(dk, dv)
+        chunked = 4 * per * max_chunks * heads <= CHANNEL_DELTA_CHUNKED_MAX_BYTES
+    if chunked:
+        per = lib.load().rlis_channel_delta_chunk_floats(dk, dv)
+        ws = torch.empty((max_chunks * heads * per,), dtype=torch.float32, device=q.device)
+        lib.call("rlis_channel_delta_chunks", out.data_ptr(), heads * dv, q.data_ptr(), k.data_ptr(),
+                 v.data_ptr(), ld, b_raw.data_ptr(), ldb, z.data_ptr(), ldz,
+                 _vec(a_log, heads, "channel_delta_scan A_log"),
+                 _vec(dt_bias, heads * dk, "channel_delta_scan dt_bias"),
+                 state.data_ptr(), stride, _meta(cu, num_seqs + 1, "cu"),
+                 _meta(slots, num_seqs, "slots"), num_seqs, heads, kv_heads, dk, dv, max_chunks,
+                 ws.data_ptr(), lib.stream_ptr())
+        return out
     lib.call("rlis_channel_delta_scan", out.data_ptr(), heads * dv, q.data_ptr(), k.data_ptr(),
              v.data_ptr(), ld, b_raw.data_ptr(), ldb, z.data_ptr(), ldz,
              _vec(a_log, heads, "channel_delta_scan A_log"),

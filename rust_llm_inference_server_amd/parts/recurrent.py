@@ -474,7 +474,8 @@ class ChannelDelta(Mixer):
         ops.tail_update(tail, p, C, self.taps - 1, cu, slots, n)
         o = ops.channel_delta_scan(qkv[:, :G * d], qkv[:, G * d:2 * G * d], qkv[:, 2 * G * d:],
                                    p[:, self.b_at:self.b_at + H], up[:, :H * d], self.a_log,
-                                   self.dt_bias, S, cu, slots, n, H, G, d, dv)
+                                   self.dt_bias, S, cu, slots, n, H, G, d, dv,
+                                   longest=getattr(step, "max_new", None))
         y = ops.head_norm_gate(o, self.norm, up[:, self.gate_at:], H, dv, self.eps, self.act_dtype,
                                sigmoid_gate=True)
         return ops.pending_linear(y, self.w_o, self.act_dtype)

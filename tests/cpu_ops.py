@@ -422,7 +422,7 @@ def delta_scan(q, k, v, b_raw, a_raw, a_log, dt_bias, state, cu, slots, num_seqs
 
 
 def channel_delta_scan(q, k, v, b_raw, z, a_log, dt_bias, state, cu, slots, num_seqs, heads,
-                       kv_heads, dk, dv, tiled=None):
+                       kv_heads, dk, dv, tiled=None, longest=None):
     T = q.shape[0]
     out = torch.empty((T, heads * dv), dtype=torch.float32)
     g = torch.nn.functional.softplus(z + dt_bias).reshape(T, heads, dk)

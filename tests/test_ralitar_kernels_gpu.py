@@ -225,13 +225,15 @@ def test_rows_behind_whole_row_norms(dtype, nh, nkv, D, real, rot, interleaved):
 
 
 # ------------------------------------------------------------------------ the recurrences
-@pytest.mark.parametrize("tiled", [False, "wide", "narrow", None])
+@pytest.mark.parametrize("tiled", [False, "wide", "narrow", None, "chunked"])
 @pytest.mark.parametrize("heads, kv_heads, dk, dv", [(4, 2, 16, 24), (2, 1, 96, 50), (3, 3, 160, 33),
                                                      (2, 2, 64, 64), (1, 1, 128, 128)])
 def test_channel_delta_scan(heads, kv_heads, dk, dv, tiled):
     """One decay per head and key channel, from near one to near zero; the state carried over
     steps with runs that end at, before and behind a tile's edge."""
     ops = _ops()
+    if tiled == "chunked" and dk > 128:
+        pytest.skip("the chunked form takes up to 128 key channels")
     g = torch.Generator().manual_seed(heads * 1000 + dk)
     totals = [sum(s[i] for s in STEPS) for i in range(3)]
     rand = lambda T, n: torch.randn(T, n, generator=g)
@@ -271,6 +273,50 @@ def test_channel_delta_scan(heads, kv_heads, dk, dv, tiled):
         assert rel(torch.cat(got[i]), want[i]) < 1e-5
     assert float((buf[1] - 7.5).abs().max()) == 0.0
     assert float((buf[:, :8] - 7.5).abs().max()) == 0.0
+
+
+@pytest.mark.parametrize("strength", [0.0, 3.0, 9.0])
+@pytest.mark.parametrize("heads, kv_heads, dk, dv", [(2, 1, 128, 128), (3, 3, 40, 70)])
+def test_long_runs_of_the_channel_delta_rule(heads, kv_heads, dk, dv, strength):
+    """Hundreds of tokens in one step beside short ones, in chunks on the matrix cores: decays that
+    hardly forget, and decays so strong that their products over a few tokens leave the float32
+    range (a single token may wipe a channel out between tokens that keep it)."""
+    ops = _ops()
+    g = torch.Generator().manual_seed(dk + int(strength))
+    lengths, slots_of = [1, 500, 65, 64, 7], [4, 0, 2, 5, 1]
+    T = sum(lengths)
+    rand = lambda *shape: torch.randn(*shape, generator=g)
+    q, k = (t / t.norm(dim=-1, keepdim=True) for t in (rand(T, kv_heads, dk), rand(T, kv_heads, dk)))
+    v, b = rand(T, heads * dv), rand(T, heads)
+    z = rand(T, heads * dk) * 2.0
+    z[torch.rand(T, heads * dk, generator=g) < 0.02] = 60.0
+    a_log, dt = torch.full((heads,), strength - 4.0), rand(heads * dk) - 2.0
+    start = rand(6, heads, dv, dk)
+    buf, state = _state(6, heads * dv * dk)
+    state.copy_(start.reshape(6, -1))
+    cu, slots, _ = _meta(lengths, slots_of)
+    qkv = torch.cat([q.reshape(T, -1), k.reshape(T, -1), v], dim=1).to(DEV)
+    n = kv_heads * dk
+    got = ops.channel_delta_scan(qkv[:, :n], qkv[:, n:2 * n], qkv[:, 2 * n:], b.to(DEV), z.to(DEV),
+                                 a_log.to(DEV), dt.to(DEV), state, cu, slots, 5, heads, kv_heads,
+                                 dk, dv, longest=max(lengths)).double().cpu()
+    dec = torch.exp(-torch.exp(a_log.double()).reshape(1, heads, 1)
+                    * plain.softplus(z.double() + dt.double()).reshape(T, heads, dk))
+    beta, at = torch.sigmoid(b.double()), 0
+    for length, slot in zip(lengths, slots_of):
+        S = start[slot].double().transpose(1, 2).clone()                     # [head][key][value]
+        for t in range(at, at + length):
+            for h in range(heads):
+                kt, qt = k[t, h // (heads // kv_heads)].double(), q[t, h // (heads // kv_heads)].double()
+                S[h] = dec[t, h].reshape(-1, 1) * S[h]
+                u = beta[t, h] * (v[t, h * dv:(h + 1) * dv].double() - S[h].T @ kt)
+                S[h] = S[h] + torch.outer(kt, u)
+                want = S[h].T @ qt
+                assert float((got[t, h * dv:(h + 1) * dv] - want).abs().max()) < 1e-4, (length, t - at)
+        left = state[slot].cpu().double().reshape(heads, dv, dk)
+        assert float((left - S.transpose(1, 2)).abs().max()) < 1e-4
+        at += length
+    assert float((state[3].cpu() - start[3].reshape(-1)).abs().max()) == 0.0
 
 
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
