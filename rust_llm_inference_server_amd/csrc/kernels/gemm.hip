@@ -997,7 +997,7 @@ __global__ __launch_bounds__(IPW == 1 ? 1024 : 512) void gemm_bf16_stream_kernel
           }
           gate *= inv_rms;
           up *= inv_rms;
-          st(y + c, gate / (1.0f + expf(-gate)) * up);
+          st(y + c, gated_result(gate, up, nm.gelu));
         }
       } else if (JOIN) {
         const long long n = (long long)tile * TR + i;
@@ -1195,7 +1195,8 @@ RLIS_API int rlis_norm_linear_max_k() { return kStreamNormMaxK; }
 
 // gated == 0: y (T, N) = x W^T (one result up to K = 8192, float32 partial results per slice
 // beyond).  gated != 0: W is (2N, K) = [Wg; Wu] and
-// y (T, N) = silu(x Wg^T) * (x Wu^T), K <= 4096.  bfloat16 operands, K a multiple of 8, up to
+// y (T, N) = silu(x Wg^T) * (x Wu^T), K <= 4096 (gated == 2: the tanh form of GELU in place of SiLU).
+// bfloat16 operands, K a multiple of 8, up to
 // rlis_gemm_bf16_stream_max_rows(K) rows (more than 16 go to the kernel of gemm_wide.hip).
 RLIS_API int rlis_gemm_bf16_stream(const void* X, const void* W, void* Y, int y_dtype, int T,
                                    int N, int K, long long ldx, long long ldw, long long ldy,
@@ -1203,6 +1204,7 @@ RLIS_API int rlis_gemm_bf16_stream(const void* X, const void* W, void* Y, int y_
   if (check_skinny("gemm_bf16_stream", X, W, T, N, K, ldx, ldw, ldy)) return 1;
   if (T > 16) {
     StreamNorm none = {};
+    none.gelu = gated == 2;
     return rlis_launch_stream_wide("gemm_bf16_stream", kStreamPlain, X, W, Y, y_dtype, T, N, K, ldx,
                                    ldw, ldy, gated, none, stream);
   }
@@ -1214,6 +1216,7 @@ RLIS_API int rlis_gemm_bf16_stream(const void* X, const void* W, void* Y, int y_
                "%d, not %d", kStreamNormMaxK, K);
   if (T == 0) return 0;
   StreamNorm nm = {};
+  nm.gelu = gated == 2;
   return dispatch_stream<kStreamPlain>("gemm_bf16_stream", X, W, Y, y_dtype, T, N, K, ldx, ldw, ldy,
                                 part_stride, gated, nm, stream);
 }

@@ -60,7 +60,15 @@ struct StreamNorm {
   const float* scale_parts;  // the same layout, scale_count entries a token
   int scale_count;
   int ss_stride;             // a multiple of 4
+  int gelu;                  // gated: the gate passes the tanh form of GELU instead of SiLU
 };
+
+// act(gate) * up of the gated form: SiLU is gate * sigmoid(gate), the tanh form of GELU is gate *
+// sigmoid(2 sqrt(2 / pi) (gate + 0.044715 gate^3)).
+__device__ __forceinline__ float gated_result(float gate, float up, int gelu) {
+  const float a = gelu ? gelu_slope(gate) * gate : gate;
+  return gate / (1.0f + expf(-a)) * up;
+}
 
 
 // What a kernel does beside the product: nothing, the fused norm (x made from the residual in

@@ -200,7 +200,7 @@ __global__ __launch_bounds__(AHEAD == 2 ? 512 : (TG == 2 ? 768 : 512)) void gemm
           }
           gate *= inv_rms;
           up *= inv_rms;
-          st(Y + (long long)tok * sh.ldy + c, gate / (1.0f + expf(-gate)) * up);
+          st(Y + (long long)tok * sh.ldy + c, gated_result(gate, up, nm.gelu));
         }
       } else if constexpr (JOIN) {
         const long long n = (long long)tile * TR + i;

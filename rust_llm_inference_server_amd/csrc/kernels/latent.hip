@@ -48,6 +48,58 @@ __global__ __launch_bounds__(256) void head_linear_kernel(
   }
 }
 
+// The same for at most 16 tokens: a workgroup's waves take 16 columns each.
+template <typename T, typename TO, bool ALIGNED>
+__global__ __launch_bounds__(256) void head_linear_few_kernel(
+    const T* __restrict__ x, long long ldx, int x_head, const T* __restrict__ w,
+    TO* __restrict__ y, long long ldy, int y_head, int rows, int N, int K) {
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  const int h = blockIdx.z;
+  const int n = blockIdx.y * 64 + wave * 16 + lane % 16;
+  if (n - lane % 16 >= N) return;
+  const T* b_row[1] = {w + ((long long)h * N + min(n, N - 1)) * K};
+  mma_f32x4 acc[1];
+  wave_tile_product<T, 1, ALIGNED>(x + (long long)min(lane % 16, rows - 1) * ldx + (long long)h * x_head,
+                                   b_row, K, acc);
+#pragma unroll
+  for (int i = 0; i < 4; ++i) {
+    const int t = (lane / 16) * 4 + i;
+    if (t < rows && n < N) st(y + (long long)t * ldy + (long long)h * y_head + n, acc[0][i]);
+  }
+}
+
+// The same with 64 tokens a wave (four blocks of 16 that share every fragment of w), for steps of
+// many rows; the sums of a row are the same bits.
+template <typename T, typename TO, bool ALIGNED>
+__global__ __launch_bounds__(256) void head_linear_rows_kernel(
+    const T* __restrict__ x, long long ldx, int x_head, const T* __restrict__ w,
+    TO* __restrict__ y, long long ldy, int y_head, int rows, int N, int K) {
+  const int wave = threadIdx.x / kWave, lane = threadIdx.x % kWave;
+  const int h = blockIdx.z;
+  const int t0 = (blockIdx.x * 4 + wave) * 64;
+  if (t0 >= rows) return;
+  const int n0 = blockIdx.y * 64;
+  const T *a_row[4], *b_row[4];
+#pragma unroll
+  for (int b = 0; b < 4; ++b) {
+    a_row[b] = x + (long long)min(t0 + b * 16 + lane % 16, rows - 1) * ldx + (long long)h * x_head;
+    b_row[b] = w + ((long long)h * N + min(n0 + b * 16 + lane % 16, N - 1)) * K;
+  }
+  mma_f32x4 acc[4][4];
+  wave_tile_product_rows<T, 4, 4, ALIGNED>(a_row, b_row, K, acc);
+#pragma unroll
+  for (int a = 0; a < 4; ++a)
+#pragma unroll
+    for (int b = 0; b < 4; ++b) {
+      const int n = n0 + b * 16 + lane % 16;
+#pragma unroll
+      for (int i = 0; i < 4; ++i) {
+        const int t = t0 + a * 16 + (lane / 16) * 4 + i;
+        if (t < rows && n < N) st(y + (long long)t * ldy + (long long)h * y_head + n, acc[a][b][i]);
+      }
+    }
+}
+
 RLIS_API int rlis_head_linear(const void* x, int dtype, long long ldx, int x_head, const void* w,
                               void* y, int y_dtype, long long ldy, int y_head, int rows, int H,
                               int N, int K, hipStream_t stream) {
@@ -57,11 +109,16 @@ RLIS_API int rlis_head_linear(const void* x, int dtype, long long ldx, int x_hea
                "head_linear: strides shorter than the heads they hold");
   RLIS_REQUIRE(H <= 65535 && ceil_div(N, 64) <= 65535, "head_linear: too many heads or columns");
   if (rows == 0) return 0;
-  dim3 grid(ceil_div(rows, 64), ceil_div(N, 64), H);
-#define LAUNCH(T, TO, AL)                                                                  \
-  head_linear_kernel<T, TO, AL><<<grid, 256, 0, stream>>>((const T*)x, ldx, x_head,        \
-                                                         (const T*)w, (TO*)y, ldy, y_head, \
-                                                         rows, N, K)
+  dim3 grid(ceil_div(rows, 64), ceil_div(N, 64), H), wide(ceil_div(rows, 256), ceil_div(N, 64), H);
+#define LAUNCH_AS(KERNEL, GRID, T, TO, AL)                                                       \
+  KERNEL<T, TO, AL><<<GRID, 256, 0, stream>>>((const T*)x, ldx, x_head, (const T*)w, (TO*)y, ldy, \
+                                              y_head, rows, N, K)
+#define LAUNCH(T, TO, AL)                                                       \
+  do {                                                                          \
+    if (rows <= 16) LAUNCH_AS(head_linear_few_kernel, grid, T, TO, AL);         \
+    else if (rows >= 512) LAUNCH_AS(head_linear_rows_kernel, wide, T, TO, AL);  \
+    else LAUNCH_AS(head_linear_kernel, grid, T, TO, AL);                        \
+  } while (0)
   if (dtype == RLIS_BF16) {
     const bool al = mma_rows_aligned<bf16_t>(x, ldx, x_head, K) &&
                     mma_rows_aligned<bf16_t>(w, K, 0, K);
@@ -75,6 +132,7 @@ RLIS_API int rlis_head_linear(const void* x, int dtype, long long ldx, int x_hea
     RLIS_REQUIRE(false, "head_linear: unknown dtype %d", dtype);
   }
 #undef LAUNCH
+#undef LAUNCH_AS
   RLIS_LAUNCH_CHECK("head_linear");
   return 0;
 }
@@ -727,11 +785,40 @@ __global__ void sigmoid_gate_kernel(TX* __restrict__ o, long long ldo, const TX*
   st(p, ld(p) / (1.0f + expf(-ld(g + t * ldg + j))));
 }
 
+// bfloat16, eight columns a thread (16-byte accesses), the hardware's exponential and reciprocal.
+__global__ void sigmoid_gate_bf16x8_kernel(bf16_t* __restrict__ o, long long ldo,
+                                           const bf16_t* __restrict__ g, long long ldg, int N8,
+                                           long long total8) {
+  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= total8) return;
+  const long long t = i / N8;
+  const int j = (int)(i % N8) * 8;
+  const uint4 ov = *(const uint4*)(o + t * ldo + j), gv = *(const uint4*)(g + t * ldg + j);
+  const uint32_t ow[4] = {ov.x, ov.y, ov.z, ov.w}, gw[4] = {gv.x, gv.y, gv.z, gv.w};
+  uint32_t r[4];
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float e0 = __builtin_amdgcn_exp2f(__uint_as_float(gw[k] << 16) * -1.4426950408889634f);
+    const float e1 = __builtin_amdgcn_exp2f(__uint_as_float(gw[k] & 0xffff0000u) * -1.4426950408889634f);
+    r[k] = (uint32_t)f32_to_bf16(__uint_as_float(ow[k] << 16) * __builtin_amdgcn_rcpf(1.0f + e0)) |
+           ((uint32_t)f32_to_bf16(__uint_as_float(ow[k] & 0xffff0000u) *
+                                  __builtin_amdgcn_rcpf(1.0f + e1)) << 16);
+  }
+  *(uint4*)(o + t * ldo + j) = make_uint4(r[0], r[1], r[2], r[3]);
+}
+
 RLIS_API int rlis_sigmoid_gate(void* o, long long ldo, const void* g, long long ldg, int dtype,
                                int T, int N, hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && N > 0 && ldo >= N && ldg >= N, "sigmoid_gate: bad sizes");
   const long long total = (long long)T * N;
   if (total == 0) return 0;
+  if (dtype == RLIS_BF16 && N % 8 == 0 && ldo % 8 == 0 && ldg % 8 == 0 && (uintptr_t)o % 16 == 0 &&
+      (uintptr_t)g % 16 == 0) {
+    sigmoid_gate_bf16x8_kernel<<<(unsigned)ceil_div_ll(total / 8, 256), 256, 0, stream>>>(
+        (bf16_t*)o, ldo, (const bf16_t*)g, ldg, N / 8, total / 8);
+    RLIS_LAUNCH_CHECK("sigmoid_gate");
+    return 0;
+  }
   const unsigned blocks = (unsigned)ceil_div_ll(total, 256);
   if (dtype == RLIS_F32)
     sigmoid_gate_kernel<float><<<blocks, 256, 0, stream>>>((float*)o, ldo, (const float*)g, ldg, N, total);

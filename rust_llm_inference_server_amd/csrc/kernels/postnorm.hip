@@ -398,6 +398,102 @@ __global__ __launch_bounds__(256) void row_prepare_kernel(
   }
 }
 
+// The usual case (bfloat16, heads of a multiple of 8, neighbouring dims as pairs, a rotated width
+// of a multiple of 8 or none): a thread owns CH pieces of eight dims and keeps them; everything
+// it reads, the weights and angles too, is asked for before the sums are waited for.
+template <int CH>
+__global__ __launch_bounds__(1024) void row_prepare_bf16x8_kernel(
+    bf16_t* __restrict__ out, const bf16_t* __restrict__ p, long long ldp, int nh, int nkv, int D,
+    int real, const float* __restrict__ bias, const float* __restrict__ q_weight,
+    const float* __restrict__ k_weight, float eps, const float* __restrict__ cos_t,
+    const float* __restrict__ sin_t, int rot, const int* __restrict__ positions) {
+  __shared__ float red[2][16];
+  const int t = blockIdx.x, NT = blockDim.x;
+  const bf16_t* row = p + (long long)t * ldp;
+  const int q_cols = nh * D, cols = (nh + nkv) * D;
+  bf16_t* dst = out + (long long)t * (cols + nkv * D);
+  uint4 raw[CH];
+  float4 b4[CH][2], w4[CH][2], c4[CH], s4[CH];
+  int at[CH];
+  const int half = rot / 2;
+  const long long angle = cos_t ? (long long)positions[t] * half : 0;
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int c = (threadIdx.x + i * NT) * 8;
+    at[i] = c < cols ? c : 0;                // (past the end: the first piece again, not used)
+    raw[i] = *(const uint4*)(row + at[i]);
+    const float* w = at[i] < q_cols ? q_weight + at[i] : k_weight + (at[i] - q_cols);
+    w4[i][0] = *(const float4*)w;
+    w4[i][1] = *(const float4*)(w + 4);
+    b4[i][0] = b4[i][1] = make_float4(0.f, 0.f, 0.f, 0.f);
+    if (bias) {                              // (the same for the whole grid)
+      b4[i][0] = *(const float4*)(bias + at[i]);
+      b4[i][1] = *(const float4*)(bias + at[i] + 4);
+    }
+    if (cos_t) {
+      const int j = at[i] % D;
+      const long long a = angle + (j < rot ? j / 2 : 0);
+      c4[i] = *(const float4*)(cos_t + a);
+      s4[i] = *(const float4*)(sin_t + a);
+    }
+  }
+  float v[CH][8];
+  float sq = 0.f, sk = 0.f;
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const uint32_t u[4] = {raw[i].x, raw[i].y, raw[i].z, raw[i].w};
+    const float b[8] = {b4[i][0].x, b4[i][0].y, b4[i][0].z, b4[i][0].w,
+                        b4[i][1].x, b4[i][1].y, b4[i][1].z, b4[i][1].w};
+    float s = 0.f;
+#pragma unroll
+    for (int e = 0; e < 8; ++e) {
+      v[i][e] = __uint_as_float(e % 2 ? u[e / 2] & 0xffff0000u : u[e / 2] << 16) + b[e];
+      s += v[i][e] * v[i][e];
+    }
+    const bool live = (int)(threadIdx.x + i * NT) * 8 < cols;
+    sq += live && at[i] < q_cols ? s : 0.f;
+    sk += live && at[i] >= q_cols ? s : 0.f;
+  }
+  sq = wave_sum(sq);
+  sk = wave_sum(sk);
+  if (threadIdx.x % kWave == 0) {
+    red[0][threadIdx.x / kWave] = sq;
+    red[1][threadIdx.x / kWave] = sk;
+  }
+  __syncthreads();
+  sq = sk = 0.f;
+  for (int w = 0; w < NT / kWave; ++w) {
+    sq += red[0][w];
+    sk += red[1][w];
+  }
+  const float q_inv = 1.0f / sqrtf(sq / (float)(nh * real) + eps);
+  const float k_inv = 1.0f / sqrtf(sk / (float)(nkv * real) + eps);
+#pragma unroll
+  for (int i = 0; i < CH; ++i) {
+    const int c = (threadIdx.x + i * NT) * 8;
+    if (c >= cols) continue;
+    const bool is_q = c < q_cols;
+    const float inv = is_q ? q_inv : k_inv;
+    if (!is_q) store_dims<bf16_t, 8>(dst + nkv * D + c, v[i]);
+    const float w[8] = {w4[i][0].x, w4[i][0].y, w4[i][0].z, w4[i][0].w,
+                        w4[i][1].x, w4[i][1].y, w4[i][1].z, w4[i][1].w};
+    float r[8];
+#pragma unroll
+    for (int e = 0; e < 8; ++e) r[e] = v[i][e] * inv * w[e];
+    if (cos_t && c % D < rot) {
+      const float cs[4] = {c4[i].x, c4[i].y, c4[i].z, c4[i].w};
+      const float sn[4] = {s4[i].x, s4[i].y, s4[i].z, s4[i].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float a = r[2 * e], b = r[2 * e + 1];
+        r[2 * e] = a * cs[e] - b * sn[e];
+        r[2 * e + 1] = b * cs[e] + a * sn[e];
+      }
+    }
+    store_dims<bf16_t, 8>(dst + c, r);
+  }
+}
+
 RLIS_API int rlis_row_prepare(void* out, const void* p, int dtype, long long ldp, int T, int nh,
                               int nkv, int D, int real, const float* bias, const float* q_weight,
                               const float* k_weight, float eps, const float* cos, const float* sin,
@@ -417,6 +513,21 @@ RLIS_API int rlis_row_prepare(void* out, const void* p, int dtype, long long ldp
   row_prepare_kernel<TX, V, INTER><<<T, 256, 0, stream>>>(                                        \
       (TX*)out, (const TX*)p, ldp, nh, nkv, D, real, bias, q_weight, k_weight, eps, cos, sin,     \
       cos ? rot : 0, positions)
+  const int pieces = (nh + nkv) * D / 8;
+  if (wide && interleaved && pieces <= 4096 && (!cos || (rot % 8 == 0 && (uintptr_t)cos % 16 == 0 &&
+                                                         (uintptr_t)sin % 16 == 0)) &&
+      (!bias || (uintptr_t)bias % 16 == 0) && (uintptr_t)q_weight % 16 == 0 && (uintptr_t)k_weight % 16 == 0) {
+#define LAUNCH8(CH)                                                                                \
+  row_prepare_bf16x8_kernel<CH><<<T, ceil_div(ceil_div(pieces, CH), 64) * 64, 0, stream>>>(         \
+      (bf16_t*)out, (const bf16_t*)p, ldp, nh, nkv, D, real, bias, q_weight, k_weight, eps, cos,    \
+      sin, cos ? rot : 0, positions)
+    if (pieces <= 512) LAUNCH8(1);
+    else if (pieces <= 1024) LAUNCH8(2);
+    else LAUNCH8(4);
+#undef LAUNCH8
+    RLIS_LAUNCH_CHECK("row_prepare");
+    return 0;
+  }
   if (interleaved) {
     RLIS_REQUIRE(D % 2 == 0, "row_prepare: pairs of neighbouring dims need an even head size");
     if (wide) LAUNCH(bf16_t, 8, true);

@@ -152,6 +152,96 @@ __global__ __launch_bounds__(256) void causal_conv_kernel(
   }
 }
 
+// The same for layouts in steps of four channels and up to five taps (what models have), without
+// rows to mix in: a thread owns four neighbouring channels of TT consecutive tokens, asks for the
+// TT + K - 1 rows they need at once and slides over them; a token whose taps reach in front of
+// the step (the same for the whole workgroup) takes those rows from the tail.  Unit groups are
+// summed over group / 4 neighbouring lanes (a power of two).  With update_tail (every sequence
+// brings one token, TT = 1) the thread also leaves the tail as tail_update would.
+template <int K, int TT, typename TO>
+__global__ __launch_bounds__(256) void causal_conv4_kernel(
+    TO* __restrict__ out, const float* __restrict__ x, long long ldx, const float* __restrict__ taps,
+    const float* __restrict__ bias, const float* __restrict__ in_bias, int C, float* state,
+    long long state_stride, const int* __restrict__ seq_of_token, const int* __restrict__ cu,
+    const int* __restrict__ slots, int T, int unit_channels, int unit_lanes, int scaled_channels,
+    float scale, float unit_eps, int activation, int update_tail) {
+  constexpr int R = K - 1;
+  const int t0 = blockIdx.x * TT;
+  const int c_own = (blockIdx.y * 256 + threadIdx.x) * 4;
+  const bool live = c_own < C;               // (lanes past the end stay for the sums over lanes)
+  const int c = live ? c_own : 0;
+  float4 rows[TT + R];
+#pragma unroll
+  for (int r = 0; r < TT + R; ++r)
+    rows[r] = *(const float4*)(x + (long long)min(max(t0 + r - R, 0), T - 1) * ldx + c);
+  float w[4 * K];                            // [channel][tap]
+#pragma unroll
+  for (int i = 0; i < K; ++i) {
+    const float4 v = *(const float4*)(taps + (long long)c * K + 4 * i);
+    w[4 * i] = v.x; w[4 * i + 1] = v.y; w[4 * i + 2] = v.z; w[4 * i + 3] = v.w;
+  }
+  float4 b = make_float4(0.f, 0.f, 0.f, 0.f);
+  if (bias) b = *(const float4*)(bias + c);
+  if (in_bias) {
+    const float4 s = *(const float4*)(in_bias + c);
+#pragma unroll
+    for (int r = 0; r < TT + R; ++r) {
+      rows[r].x += s.x; rows[r].y += s.y; rows[r].z += s.z; rows[r].w += s.w;
+    }
+  }
+#pragma unroll
+  for (int k = 0; k < TT; ++k) {
+    const int t = t0 + k;
+    if (t >= T) break;
+    const int s = seq_of_token[t];
+    const int rel = t - cu[s];
+    float* tail = state + (long long)slots[s] * state_stride + c;
+    float4 in[K];
+#pragma unroll
+    for (int j = 0; j < K; ++j) in[j] = rows[k + j];
+    if (rel < R) {
+#pragma unroll
+      for (int j = 0; j < R; ++j)
+        if (R - j > rel) in[j] = *(const float4*)(tail + (long long)(j + rel) * C);
+    }
+    if (update_tail && live) {
+#pragma unroll
+      for (int j = 0; j < R; ++j) *(float4*)(tail + (long long)j * C) = in[j + 1];
+    }
+    float y[4] = {b.x, b.y, b.z, b.w};
+#pragma unroll
+    for (int j = 0; j < K; ++j) {
+      y[0] += w[j] * in[j].x;
+      y[1] += w[K + j] * in[j].y;
+      y[2] += w[2 * K + j] * in[j].z;
+      y[3] += w[3 * K + j] * in[j].w;
+    }
+    if (activation) {
+#pragma unroll
+      for (int e = 0; e < 4; ++e) y[e] = siluf_(y[e]);
+    }
+    if (unit_channels) {                     // (the same for the whole grid)
+      float ss = (y[0] * y[0] + y[1] * y[1]) + (y[2] * y[2] + y[3] * y[3]);
+      for (int o = 1; o < unit_lanes; o *= 2) ss += __shfl_xor(ss, o, kWave);
+      if (c_own < unit_channels) {
+        const float mult = 1.0f / sqrtf(ss + unit_eps) * (c_own < scaled_channels ? scale : 1.0f);
+#pragma unroll
+        for (int e = 0; e < 4; ++e) y[e] *= mult;
+      }
+    }
+    if (!live) continue;
+    TO* o = out + (long long)t * C + c;
+    if constexpr (sizeof(TO) == 4) {
+      *(float4*)o = make_float4(y[0], y[1], y[2], y[3]);
+    } else {
+      uint2 v;
+      v.x = (uint32_t)f32_to_bf16(y[0]) | ((uint32_t)f32_to_bf16(y[1]) << 16);
+      v.y = (uint32_t)f32_to_bf16(y[2]) | ((uint32_t)f32_to_bf16(y[3]) << 16);
+      *(uint2*)o = v;
+    }
+  }
+}
+
 // ------------------------------------------------------------------ the two scans
 // A wave walks kCols value channels of one (sequence, head): lane i holds S[i][j] of each (and
 // i + 64, ... for more than 64 key channels), so what a token brings per key channel is loaded
@@ -821,12 +911,12 @@ RLIS_API int rlis_tail_update(float* state, long long state_stride, const void* 
 
 RLIS_API int rlis_causal_conv(void* out, int out_dtype, const float* x, long long ldx, const float* taps,
                               const float* bias, const float* in_bias, int C, int K,
-                              const float* state, long long state_stride,
+                              float* state, long long state_stride,
                               const int* seq_of_token, const int* cu, const int* slots, int T,
                               int unit_channels, int unit_group, int scaled_channels, float scale,
                               float unit_eps, int rest_group, int activation, const void* blend,
                               long long ld_blend, int blend_from, float blend_weight,
-                              hipStream_t stream) {
+                              int update_tail, hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && C > 0 && K >= 1 && K <= 16, "causal_conv: bad sizes T=%d C=%d taps=%d", T, C, K);
   RLIS_REQUIRE(!blend || (blend_from >= 0 && blend_from < C && ld_blend >= C - blend_from),
                "causal_conv: the rows to mix in do not cover channels %d to %d", blend_from, C);
@@ -840,6 +930,42 @@ RLIS_API int rlis_causal_conv(void* out, int out_dtype, const float* x, long lon
   RLIS_REQUIRE(unit_channels == C || (rest_group > 0 && rest_group <= 1024),
                "causal_conv: bad group size %d for the other channels", rest_group);
   if (T == 0) return 0;
+  const int lanes = unit_channels ? unit_group / 4 : 1;
+  if (!blend && K <= 5 && C % 4 == 0 && ldx % 4 == 0 && state_stride % 4 == 0 &&
+      (uintptr_t)x % 16 == 0 && (uintptr_t)state % 16 == 0 && (uintptr_t)out % 16 == 0 &&
+      (uintptr_t)taps % 16 == 0 && (uintptr_t)bias % 16 == 0 && (uintptr_t)in_bias % 16 == 0 &&
+      (unit_channels == 0 || (unit_group % 4 == 0 && lanes <= kWave && (lanes & (lanes - 1)) == 0 &&
+                              scaled_channels % 4 == 0))) {
+    RLIS_REQUIRE(ceil_div(C, 1024) <= 65535, "causal_conv: too many channels");
+#define LAUNCH4(K_, TT_, TO)                                                                       \
+  causal_conv4_kernel<K_, TT_, TO><<<dim3(ceil_div(T, TT_), ceil_div(C, 1024)), 256, 0, stream>>>(  \
+      (TO*)out, x, ldx, taps, bias, in_bias, C, state, state_stride, seq_of_token, cu, slots, T,    \
+      unit_channels, lanes, scaled_channels, scale, unit_eps, activation, update_tail)
+#define BY_TOKENS(K_, TO)                                       \
+  do {                                                          \
+    if (T >= 512 && !update_tail) LAUNCH4(K_, 4, TO);           \
+    else LAUNCH4(K_, 1, TO);                                    \
+  } while (0)
+#define BY_TAPS(TO)                          \
+  do {                                       \
+    switch (K) {                             \
+      case 1: BY_TOKENS(1, TO); break;       \
+      case 2: BY_TOKENS(2, TO); break;       \
+      case 3: BY_TOKENS(3, TO); break;       \
+      case 4: BY_TOKENS(4, TO); break;       \
+      default: BY_TOKENS(5, TO); break;      \
+    }                                        \
+  } while (0)
+    if (out_dtype == RLIS_F32) BY_TAPS(float);
+    else if (out_dtype == RLIS_BF16) BY_TAPS(bf16_t);
+    else RLIS_REQUIRE(false, "causal_conv: unknown dtype %d", out_dtype);
+#undef BY_TAPS
+#undef BY_TOKENS
+#undef LAUNCH4
+    RLIS_LAUNCH_CHECK("causal_conv");
+    return 0;
+  }
+  RLIS_REQUIRE(!update_tail, "causal_conv: this layout leaves the tail to tail_update");
   const int groups = (unit_channels ? unit_channels / unit_group : 0) +
                      (unit_channels < C ? ceil_div(C - unit_channels, rest_group) : 0);
   RLIS_REQUIRE(ceil_div(groups, 4) <= 65535, "causal_conv: too many groups");

@@ -1016,10 +1016,24 @@ def linear_swiglu(x: torch.Tensor, w_gate_up: torch.Tensor) -> torch.Tensor:
 
 
 def linear_geglu(x: torch.Tensor, w_gate_up: torch.Tensor) -> torch.Tensor:
-    """``gelu(x @ Wg.T) * (x @ Wu.T)`` (tanh form) for ``w_gate_up = [Wg; Wu]`` of ``(2 I, K)``."""
-    if w_gate_up.shape[0] % 2:
+    """``gelu(x @ Wg.T) * (x @ Wu.T)`` (tanh form) for ``w_gate_up = [Wg; Wu]`` of ``(2 I, K)``: one
+    kernel where the streaming product takes the rows (as ``linear_swiglu``), else the product and
+    the GEGLU kernel."""
+    T, K = x.shape
+    two_i = w_gate_up.shape[0]
+    if two_i % 2:
         raise KernelError("linear_geglu: the fused weight needs an even number of rows")
-    return geglu(linear(x, w_gate_up, x.dtype))
+    ldx = _rows_contig(x, "linear_geglu x")
+    ldw = _rows_contig(w_gate_up, "linear_geglu weight")
+    if not (x.dtype == torch.bfloat16 and w_gate_up.dtype == torch.bfloat16
+            and K == w_gate_up.shape[1] and K % 8 == 0 and ldx % 8 == 0 and ldw % 8 == 0
+            and x.data_ptr() % 16 == 0 and w_gate_up.data_ptr() % 16 == 0
+            and 0 < T <= stream_rows(K) and _one_item_per_wave(K)):
+        return geglu(linear(x, w_gate_up, x.dtype))
+    y = torch.empty((T, two_i // 2), dtype=torch.bfloat16, device=x.device)
+    lib.call("rlis_gemm_bf16_stream", x.data_ptr(), w_gate_up.data_ptr(), y.data_ptr(), 1, T,
+             two_i // 2, K, ldx, ldw, two_i // 2, 0, 2, lib.stream_ptr())
+    return y
 
 
 # ------------------------------------------------------------ rotation + cache write

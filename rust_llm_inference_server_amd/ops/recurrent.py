@@ -115,7 +115,7 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor,
                 out_dtype: torch.dtype = torch.float32, activation: bool = True,
                 blend: Optional[torch.Tensor] = None, blend_from: int = 0,
                 blend_weight: float = 0.0,
-                in_bias: Optional[torch.Tensor] = None) -> torch.Tensor:
+                in_bias: Optional[torch.Tensor] = None, keep_tail: bool = False) -> torch.Tensor:
     """``silu`` of the causal convolution over time of the first ``C`` columns of ``x`` (float32)
     with ``taps (C, K)`` (the last column multiplies the current row; the ``K - 1`` rows in
     front of the step come from ``state``), plus ``bias (C)`` under the ``silu`` when given
@@ -125,7 +125,9 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor,
     ``out_dtype``, ``C - blend_from`` columns) the channels from ``blend_from`` on become
     ``(1 - blend_weight) * y + blend_weight * blend``.  Channels below ``unit_channels`` are then made
     unit vectors in groups of ``unit_group``: ``y / sqrt(sum y^2 + unit_eps)``, those below
-    ``scaled_channels`` times ``scale``.  Returns ``(T, C)`` in ``out_dtype`` (float32 arithmetic)."""
+    ``scaled_channels`` times ``scale``.  Returns ``(T, C)`` in ``out_dtype`` (float32 arithmetic).
+    ``keep_tail``: ``state`` is left as ``tail_update`` leaves it, by the same kernel where every
+    sequence brings one token and the layout goes in steps of four channels."""
     ldx = _rows(x, "causal_conv x", torch.float32)
     C, K = taps.shape
     _vec(taps.reshape(-1), C * K, "causal_conv taps")
@@ -141,6 +143,11 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor,
             raise KernelError(f"causal_conv: rows to mix in of shape {tuple(blend.shape)} for "
                               f"channels {blend_from} to {C} of {T} tokens")
         blend_ptr = blend.data_ptr()
+    by_four = (blend is None and K <= 5 and all(
+        n % 4 == 0 for n in (C, ldx, stride, unit_group if unit_channels else 0, scaled_channels))
+        and (not unit_channels or (unit_group <= 256 and unit_group & (unit_group - 1) == 0))
+        and all(v is None or v.data_ptr() % 16 == 0 for v in (x, taps, state, bias, in_bias)))
+    fused = keep_tail and by_four and num_seqs == T
     lib.call("rlis_causal_conv", out.data_ptr(), _DT[out_dtype], x.data_ptr(), ldx,
              taps.data_ptr(), None if bias is None else _vec(bias, C, "causal_conv bias"),
              None if in_bias is None else _vec(in_bias, C, "causal_conv input bias"), C, K,
@@ -148,7 +155,9 @@ def causal_conv(x: torch.Tensor, taps: torch.Tensor, state: torch.Tensor,
              _meta(cu, num_seqs + 1, "cu"), _meta(slots, num_seqs, "slots"), T,
              int(unit_channels), int(unit_group), int(scaled_channels), float(scale),
              float(unit_eps), int(rest_group), int(bool(activation)), blend_ptr, ld_blend,
-             int(blend_from), float(blend_weight), lib.stream_ptr())
+             int(blend_from), float(blend_weight), int(fused), lib.stream_ptr())
+    if keep_tail and K > 1 and not fused:
+        tail_update(state, x, C, K - 1, cu, slots, num_seqs, bias=in_bias)
     return out
 
 

@@ -210,8 +210,8 @@ class GatedDelta(Mixer):
              else ops.linear_f32(x, self.w_in))                           # (T, q|k|v|g|b|a)
         qkv = ops.causal_conv(p, self.conv_w, tail, step.seq_of_token, cu, slots, n,
                               unit_channels=2 * G * d, unit_group=d, scaled_channels=G * d,
-                              scale=d ** -0.5, unit_eps=self.UNIT_EPS, rest_group=dv)
-        ops.tail_update(tail, p, C, self.taps - 1, cu, slots, n)
+                              scale=d ** -0.5, unit_eps=self.UNIT_EPS, rest_group=dv,
+                              keep_tail=True)
         c = self.cols
         o = ops.delta_scan(qkv[:, :G * d], qkv[:, G * d:2 * G * d], qkv[:, 2 * G * d:],
                            p[:, c["b"]:c["b"] + H], p[:, c["a"]:c["a"] + H], self.a_log,
@@ -274,8 +274,7 @@ class SelectiveScan(Mixer):
         cu, slots, n = step.cu_seqlens, step.state_slots, step.num_seqs
         xz = ops.linear_f32(x, self.w_in)                                  # (T, x | z)
         xc = ops.causal_conv(xz, self.conv_w, tail, step.seq_of_token, cu, slots, n,
-                             bias=self.conv_b, out_dtype=self.act_dtype)
-        ops.tail_update(tail, xz, C, self.taps - 1, cu, slots, n)
+                             bias=self.conv_b, out_dtype=self.act_dtype, keep_tail=True)
         low = ops.linear_f32(xc, self.w_x)                                 # (T, dt | B | C)
         dt_raw = ops.linear(low[:, :rank], self.w_dt, torch.float32)
         y = ops.selective_scan(xc, dt_raw, self.dt_bias, low[:, rank:rank + N],
@@ -470,8 +469,8 @@ class ChannelDelta(Mixer):
         up = ops.linear_f32(ops.linear(x, self.w_low, self.act_dtype), self.w_up)
         qkv = ops.causal_conv(p, self.conv_w, tail, step.seq_of_token, cu, slots, n,
                               unit_channels=2 * G * d, unit_group=d, scaled_channels=G * d,
-                              scale=d ** -0.5, unit_eps=self.UNIT_EPS, rest_group=min(dv, 1024))
-        ops.tail_update(tail, p, C, self.taps - 1, cu, slots, n)
+                              scale=d ** -0.5, unit_eps=self.UNIT_EPS, rest_group=min(dv, 1024),
+                              keep_tail=True)
         o = ops.channel_delta_scan(qkv[:, :G * d], qkv[:, G * d:2 * G * d], qkv[:, 2 * G * d:],
                                    p[:, self.b_at:self.b_at + H], up[:, :H * d], self.a_log,
                                    self.dt_bias, S, cu, slots, n, H, G, d, dv,
@@ -557,8 +556,7 @@ class RGLRU(Mixer):
         p = ops.linear_f32(x, self.w_in)                                   # (T, x | y)
         u = ops.causal_conv(p, self.conv_w, tail, step.seq_of_token, cu, slots, num,
                             bias=self.conv_b, out_dtype=self.act_dtype, activation=False,
-                            in_bias=self.x_bias)
-        ops.tail_update(tail, p, C, self.taps - 1, cu, slots, num, bias=self.x_bias)
+                            in_bias=self.x_bias, keep_tail=True)
         gates = ops.head_linear(u, self.w_gates, n, out_dtype=torch.float32)
         y = ops.rglru_scan(u, gates, self.r_bias, self.i_bias, self.rate,
                            p[:, self.y_at:self.y_at + C], self.y_bias, S, cu, slots, num,

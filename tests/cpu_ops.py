@@ -229,8 +229,9 @@ def tail_update(state, x, channels, rows, cu, slots, num_seqs, bias=None):
 def causal_conv(x, taps, state, seq_of_token, cu, slots, num_seqs, unit_channels=0, unit_group=0,
                 scaled_channels=0, scale=1.0, unit_eps=0.0, rest_group=256, bias=None,
                 out_dtype=torch.float32, activation=True, blend=None, blend_from=0,
-                blend_weight=0.0, in_bias=None):
+                blend_weight=0.0, in_bias=None, keep_tail=False):
     C, K = taps.shape
+    raw = x
     if in_bias is not None:
         x = x[:, :C] + in_bias
     out = torch.empty((x.shape[0], C), dtype=torch.float32)
@@ -248,6 +249,8 @@ def causal_conv(x, taps, state, seq_of_token, cu, slots, num_seqs, unit_channels
         y = y / torch.sqrt((y * y).sum(-1, keepdim=True) + unit_eps)
         out[:, :unit_channels] = y.reshape(x.shape[0], unit_channels)
         out[:, :scaled_channels] *= scale
+    if keep_tail and K > 1:
+        tail_update(state, raw, C, K - 1, cu, slots, num_seqs, bias=in_bias)
     return out.to(out_dtype)
 
 

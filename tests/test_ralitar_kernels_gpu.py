@@ -130,7 +130,7 @@ def test_geglu_and_the_token_input(dtype):
         want = plain.gelu_tanh(gu[:, :I].double()) * gu[:, I:].double()
         assert rel(ops.geglu(gu.to(DEV)), want) < tol
     for T, W, I in ((1, 96, 40), (7, 256, 64), (16, 2048, 512), (21, 1024, 256), (50, 512, 128),
-                    (3, 50, 30)):
+                    (3, 50, 30), (25, 512, 48), (32, 2048, 80)):
         x = torch.randn(T, W, generator=g).to(dtype)
         w = (torch.randn(2 * I, W, generator=g) * W ** -0.5).to(dtype)
         gu = x.double() @ w.double().T
@@ -181,7 +181,9 @@ def test_pair_table_over_steps(dtype, buckets, mul_prev, mul_cur):
 @pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
 @pytest.mark.parametrize("nh, nkv, D, real, rot", [(4, 2, 16, 16, 12), (3, 1, 48, 36, 36),
                                                    (8, 2, 64, 64, 64), (2, 2, 128, 128, 32),
-                                                   (5, 5, 6, 6, 4), (1, 1, 32, 20, 0)])
+                                                   (5, 5, 6, 6, 4), (1, 1, 32, 20, 0),
+                                                   (40, 8, 128, 128, 128), (60, 20, 160, 152, 8),
+                                                   (96, 32, 256, 256, 256)])
 @pytest.mark.parametrize("interleaved", [True, False])
 def test_rows_behind_whole_row_norms(dtype, nh, nkv, D, real, rot, interleaved):
     """Biases, norms over whole rows, both rotation layouts, values as the keys in front of the
@@ -407,3 +409,77 @@ def test_convolution_with_a_bias_on_its_inputs(K):
     for i in range(3):
         want = plain.short_conv(data[i][:, :C].double() + in_bias.double(), taps.double(), bias.double())
         assert rel(torch.cat(got[i]), want) < 1e-6
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("K", [1, 2, 3, 4, 5])
+def test_convolution_that_keeps_its_tail(K, dtype):
+    """Layouts in steps of four channels, and one that is not: portions long and short, steps in
+    which every sequence brings one token, unit vectors over 4 to 256 channels; the rows left for
+    the next step are those of the separate update, bit for bit."""
+    ops = _ops()
+    steps = [[1, 1, 1], [2, 700, 5], [1, 1, 1], [1, 1, 1], [K, 1, 3], [1, 1, 1]]
+    for unit_group, heads, rest, extra in ((4, 6, 20, 4), (64, 3, 1100, 0), (256, 2, 36, 8),
+                                           (0, 0, 36, 4), (48, 2, 8, 4), (16, 2, 9, 3)):
+        U, C = unit_group * heads, unit_group * heads + rest
+        g = torch.Generator().manual_seed(K * 1000 + C)
+        totals = [sum(s[i] for s in steps) for i in range(3)]
+        xs = [torch.randn(T, C + extra, generator=g) for T in totals]
+        taps, bias, in_bias = (torch.randn(C, K, generator=g), torch.randn(C, generator=g),
+                               torch.randn(C, generator=g))
+        scaled = heads // 2 * unit_group
+        want = []
+        for x in xs:
+            y = plain.short_conv(x[:, :C].double() + in_bias.double(), taps.double(), bias.double())
+            y = y * torch.sigmoid(y)
+            if U:
+                u = y[:, :U].reshape(-1, heads, unit_group)
+                u = (u / torch.sqrt((u * u).sum(-1, keepdim=True) + 1e-6)).reshape(-1, U)
+                u[:, :scaled] *= 0.3
+                y = torch.cat([u, y[:, U:]], 1)
+            want.append(y)
+        width = max(4, C * (K - 1))
+        states = []
+        for _ in range(2):
+            buf = torch.full((4, width + 4), 7.5, device=DEV)
+            state = buf[:, :width]
+            state[SLOTS] = 0.0
+            states.append((buf, state))
+        for step, lengths in enumerate(steps):
+            cu, slots, seq = _meta(lengths, SLOTS)
+            x = torch.cat([xs[i][_cut(None, steps, step, i)] for i in range(3)]).to(DEV)
+            outs = []
+            for (_, state), keep in zip(states, (True, False)):
+                outs.append(ops.causal_conv(
+                    x, taps.to(DEV), state, seq, cu, slots, 3, unit_channels=U,
+                    unit_group=unit_group, scaled_channels=scaled, scale=0.3, unit_eps=1e-6,
+                    rest_group=64, bias=bias.to(DEV), in_bias=in_bias.to(DEV), out_dtype=dtype,
+                    keep_tail=keep))
+            if K > 1:
+                ops.tail_update(states[1][1], x, C, K - 1, cu, slots, 3, bias=in_bias.to(DEV))
+            assert torch.equal(outs[0], outs[1]) and torch.equal(states[0][0], states[1][0])
+            for i, part in enumerate(outs[0].cpu().split(lengths)):
+                ref = want[i][_cut(None, steps, step, i)]
+                tol = 1e-5 if dtype == torch.float32 else 1e-2
+                assert torch.allclose(part.double(), ref, rtol=tol, atol=tol)
+        assert float(states[0][0][1].min()) == 7.5
+
+
+@pytest.mark.parametrize("dtype", [torch.float32, torch.bfloat16])
+@pytest.mark.parametrize("N, K", [(100, 72), (40, 128), (64, 30)])
+def test_products_per_head_by_number_of_rows(dtype, N, K):
+    """Rows on both sides of every form's edge agree with the same rows alone."""
+    ops = _ops()
+    H, T = 3, 600
+    g = torch.Generator().manual_seed(N)
+    x = torch.randn(T, H * K, generator=g).to(dtype)
+    w = (torch.randn(H, N, K, generator=g) * K ** -0.5).to(dtype)
+    want = torch.matmul(x.double().reshape(T, H, K).transpose(0, 1).contiguous(),
+                        w.double().transpose(1, 2).contiguous()).transpose(0, 1).reshape(T, H * N)
+    whole = ops.head_linear(x.to(DEV), w.to(DEV), K, out_dtype=torch.float32)
+    assert rel(whole, want) < (2e-6 if dtype == torch.float32 else 5e-3)
+    for rows in (1, 16, 17, 64, 65, 256, 511, 512, 513):
+        part = ops.head_linear(x[:rows].to(DEV), w.to(DEV), K, out_dtype=torch.float32)
+        assert rel(part, want[:rows]) < (2e-6 if dtype == torch.float32 else 5e-3)
+        if dtype == torch.bfloat16:
+            assert torch.equal(part, whole[:rows])
