@@ -111,7 +111,14 @@ CONFIG_D = _model(200, 128, 1e-6, [
     _attention(2, 2, 128, 0.09, 500, (32, 500000.0), 30.0, 128),
     _delta(2, 2, 128, 96, 3, (24, 8), None),
 ], bigram=(300, 17, 5), side=32)
-CONFIGS = {"a": CONFIG_A, "b": CONFIG_B, "c": CONFIG_C, "d": CONFIG_D}
+# Recurrent layers only: nothing is paged.  Layouts in steps of four channels.
+CONFIG_E = _model(80, 32, 1e-5, [
+    _rglru(48, 2, 2, 40),
+    _delta(4, 4, 8, 16, 4, (5, 6), None),
+    _rglru(64, 4, 4, None),
+    _delta(2, 1, 32, 36, 5, (4, 9), 30),
+], bigram=(41, 13, 29))
+CONFIGS = {"a": CONFIG_A, "b": CONFIG_B, "c": CONFIG_C, "d": CONFIG_D, "e": CONFIG_E}
 
 
 def spec_of(config: dict):

@@ -199,7 +199,7 @@ def test_the_plain_implementation_does_not_look_ahead():
 
 
 # --------------------------------------------------------------------- the step function
-@pytest.mark.parametrize("name", ["a", "b", "c"])
+@pytest.mark.parametrize("name", ["a", "b", "c", "e"])
 def test_whole_prompts_and_first_tokens(backend, dtype, name, tmp_path_factory):
     folder, cfg, stored = model_case(name, dtype, tmp_path_factory)
     reqs = traces.random_requests(cfg["vocab"], [1, 2, 3, 19, 70], seed=11)
@@ -207,7 +207,7 @@ def test_whole_prompts_and_first_tokens(backend, dtype, name, tmp_path_factory):
     check_trace(runner_for(folder, backend, dtype), steps, reqs, cfg, stored, dtype)
 
 
-@pytest.mark.parametrize("name", ["a", "b", "c"])
+@pytest.mark.parametrize("name", ["a", "b", "c", "e"])
 def test_decoding_token_by_token_equals_the_prompt_pass(backend, dtype, name, tmp_path_factory):
     """One request decoded from its first token on, one after a prompt, so that chunks begin
     inside decoded tokens; single tokens go through captured steps on the GPU."""
@@ -221,7 +221,7 @@ def test_decoding_token_by_token_equals_the_prompt_pass(backend, dtype, name, tm
     check_trace(runner_for(folder, backend, dtype), steps + more, reqs, cfg, stored, dtype)
 
 
-@pytest.mark.parametrize("name", ["a", "b", "c"])
+@pytest.mark.parametrize("name", ["a", "b", "c", "e"])
 def test_portions_of_any_size(backend, dtype, name, tmp_path_factory):
     """Portions of 7, 2, 16, 3, 24, 2, 33, ... tokens: portions that end inside a page, inside a
     chunk and inside the convolutions' reach, each starting behind a token of the one before."""
@@ -231,7 +231,7 @@ def test_portions_of_any_size(backend, dtype, name, tmp_path_factory):
     check_trace(runner_for(folder, backend, dtype), steps, reqs, cfg, stored, dtype)
 
 
-@pytest.mark.parametrize("name", ["a", "c"])
+@pytest.mark.parametrize("name", ["a", "c", "e"])
 def test_mixed_batches_reuse_pages_and_slots(backend, dtype, name, tmp_path_factory):
     """Seven unequal requests through three slots and a pool that holds three of them: portions
     beside single tokens, requests left out of steps, pages and slots of finished requests taken
@@ -596,9 +596,10 @@ def test_a_fork_takes_the_state_along(backend, dtype, tmp_path_factory):
 
 
 @pytest.mark.gpu
-@pytest.mark.parametrize("dtype_name", ["float32", "bfloat16"])
-def test_the_replay_program_runs_the_model(dtype_name, tmp_path_factory, tmp_path):
-    folder, cfg, stored = model_case("a", dtype_name, tmp_path_factory)
+@pytest.mark.parametrize("name, dtype_name", [("a", "float32"), ("a", "bfloat16"),
+                                              ("e", "bfloat16")])
+def test_the_replay_program_runs_the_model(name, dtype_name, tmp_path_factory, tmp_path):
+    folder, cfg, stored = model_case(name, dtype_name, tmp_path_factory)
     reqs = traces.random_requests(cfg["vocab"], [40, 7, 25, 33, 18], seed=19)
     steps, peak = traces.trace_mixed(reqs, live=4, seed=3)
     out = traces.replay_program(folder, dtype_name, steps, peak, str(tmp_path / "out"),
