@@ -8,6 +8,7 @@
 // at slot = table[pos / page] * page + pos % page before attention reads them
 // (crates/model/src/paged.rs:258-263, 324-337).
 #include "common.h"
+#include "kv_write.h"
 
 static thread_local char g_err[512] = "";
 
@@ -831,26 +832,6 @@ __global__ void rope_kv_write_kernel(TX* __restrict__ qkv, long long row_stride,
 // first_head on: nh when q is left alone); the others take kRopeTokV tokens times kRopeVCols value columns each and turn them through LDS, so
 // that lanes which are neighbours in a page's (d, offset) layout store neighbouring offsets
 // (tokens with adjacent slots fill whole 32-byte runs, whatever their alignment).
-constexpr int kRopeTokV = 16;
-constexpr int kRopeVCols = 256;                // v columns per workgroup
-constexpr int kRopeVRow = kRopeVCols + 8;      // padded: rows stay 16-byte aligned, banks spread
-
-__device__ __forceinline__ void unpack8(const uint4 u, float (&v)[8]) {
-  const uint32_t w[4] = {u.x, u.y, u.z, u.w};
-#pragma unroll
-  for (int i = 0; i < 4; ++i) {
-    v[2 * i] = __uint_as_float(w[i] << 16);
-    v[2 * i + 1] = __uint_as_float(w[i] & 0xffff0000u);
-  }
-}
-__device__ __forceinline__ uint4 pack8(const float (&v)[8]) {
-  uint32_t w[4];
-#pragma unroll
-  for (int i = 0; i < 4; ++i)
-    w[i] = (uint32_t)f32_to_bf16(v[2 * i]) | ((uint32_t)f32_to_bf16(v[2 * i + 1]) << 16);
-  return make_uint4(w[0], w[1], w[2], w[3]);
-}
-
 __global__ __launch_bounds__(256) void rope_kv_write_bf16x8_kernel(
     bf16_t* __restrict__ qkv, long long row_stride, int k_off, int v_off, int T, int nh, int nkv,
     int d, int rot_dim, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
@@ -910,35 +891,8 @@ __global__ __launch_bounds__(256) void rope_kv_write_bf16x8_kernel(
     }
     return;
   }
-  // Values: a tile of kRopeTokV tokens times kRopeVCols columns per workgroup.
-  __shared__ __attribute__((aligned(16))) bf16_t v_s[kRopeTokV * kRopeVRow];
-  __shared__ long long page_s[kRopeTokV];                // -1: the token is not stored
-  __shared__ int off_s[kRopeTokV];
-  const int cols = nkv * d;
-  const int chunks = (cols + kRopeVCols - 1) / kRopeVCols;
-  const int vb = (int)blockIdx.x - qk_blocks;
-  const int t0 = (vb / chunks) * kRopeTokV, c0 = (vb % chunks) * kRopeVCols;
-  if (tid < kRopeTokV) {
-    const int slot = t0 + tid < T ? slots[t0 + tid] : -1;
-    const int page = slot < 0 ? -1 : slot / page_size;
-    page_s[tid] = page;
-    off_s[tid] = slot < 0 ? 0 : slot - page * page_size;
-  }
-  const int nc = min(kRopeVCols, cols - c0), nc8 = nc / 8;
-  for (int i = tid; i < kRopeTokV * nc8; i += blockDim.x) {
-    const int tt = i / nc8, c = (i - tt * nc8) * 8;
-    if (t0 + tt < T)
-      *(uint4*)(v_s + tt * kRopeVRow + c) =
-          *(const uint4*)(qkv + (long long)(t0 + tt) * row_stride + v_off + c0 + c);
-  }
-  __syncthreads();
-  for (int i = tid; i < kRopeTokV * nc; i += blockDim.x) {
-    const int tt = i % kRopeTokV, c = i / kRopeTokV;
-    const long long page = page_s[tt];
-    if (page < 0) continue;
-    const int col = c0 + c, h = col / d, j = col - h * d;
-    v_pages[((page * nkv + h) * d + j) * page_size + off_s[tt]] = v_s[tt * kRopeVRow + c];
-  }
+  store_value_tile(qkv, row_stride, v_off, T, nkv, d, slots, v_pages, page_size,
+                   (int)blockIdx.x - qk_blocks);
 }
 
 RLIS_API int rlis_rope_kv_write(void* qkv, int dtype, long long row_stride, int k_off, int v_off,

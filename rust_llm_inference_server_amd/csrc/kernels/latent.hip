@@ -140,22 +140,56 @@ RLIS_API int rlis_head_linear(const void* x, int dtype, long long ldx, int x_hea
 // ------------------------------------------------- norm, rotation and cache write
 // Per token: c = x[:R] / sqrt(mean(x[:R]^2) + eps) * weight goes to the token's cache row, the
 // r numbers behind it are rotated by the token's position (the first rot of them: entry i with
-// entry i + rot/2; the rest pass) and follow c in the row; the last r numbers of every query
-// head are rotated the same way into the head's row of q_out behind its first R columns.
+// entry i + rot/2, or with `interleaved` entry 2i with 2i + 1; the rest pass) and follow c in the
+// row; the last r numbers of every query head are rotated the same way into the head's row of
+// q_out behind its first R columns (q null: there are no queries to turn).
 // x is float32; angles come from float32 tables (positions, rot/2).  With pages_t the latent is
 // stored a second time with the positions of a page innermost ([page][j][offset]), which is how
 // the matrix-core kernel reads it as values.
+// With cq (a second row of workgroups) the latent of the queries, float32 like x, is normed by
+// the same rule into cq_out: cq[:Rq] / sqrt(mean(cq[:Rq]^2) + eps) * cq_weight.
+struct LatentQuery {
+  const float* x;        // rows ld apart; null: there is none
+  long long ld;
+  int R;
+  const float* weight;
+  void* out;             // (T, R) contiguous
+};
+
+// entry j of a rotated vector whose entries `at` hands out
+template <typename F>
+__device__ __forceinline__ float turned(F at, int j, int rot, bool interleaved,
+                                        const float* cos_r, const float* sin_r) {
+  if (j >= rot) return at(j);
+  const int half = rot / 2;
+  const int i = interleaved ? j / 2 : (j < half ? j : j - half);
+  const bool first = interleaved ? j % 2 == 0 : j < half;
+  const float u = at(interleaved ? 2 * i : i), w = at(interleaved ? 2 * i + 1 : i + half);
+  const float c = cos_r[i], s = sin_r[i];
+  return first ? u * c - w * s : w * c + u * s;
+}
+
 template <typename TX>
 __global__ __launch_bounds__(256) void latent_write_kernel(
     const float* __restrict__ x, long long ldx, const float* __restrict__ weight, float eps,
     int R, int r, int rot, const float* __restrict__ cos_t, const float* __restrict__ sin_t,
     const int* __restrict__ positions, const int* __restrict__ slots, TX* __restrict__ pages,
     TX* __restrict__ pages_t, int page_size, int write, const TX* __restrict__ q, long long ldq, int q_head, int q_off,
-    TX* __restrict__ q_out, long long ldo, int o_head, int H) {
+    TX* __restrict__ q_out, long long ldo, int o_head, int H, int interleaved, const LatentQuery cq) {
   __shared__ float red[4];
   const int t = blockIdx.x;
-  const int pos = positions[t];
+  if (blockIdx.y == 1) {
+    const float* row = cq.x + (long long)t * cq.ld;
+    TX* out = (TX*)cq.out + (long long)t * cq.R;
+    float ss = 0.f;
+    for (int j = threadIdx.x; j < cq.R; j += 256) ss += row[j] * row[j];
+    const float mult = 1.0f / sqrtf(block_sum<256>(ss, red) / (float)cq.R + eps);
+    for (int j = threadIdx.x; j < cq.R; j += 256) st(out + j, row[j] * mult * cq.weight[j]);
+    return;
+  }
   const int half = rot / 2;
+  const float* cos_r = cos_t + (rot ? (long long)positions[t] * half : 0);
+  const float* sin_r = sin_t + (rot ? (long long)positions[t] * half : 0);
   const float* xr = x + (long long)t * ldx;
   if (write) {
     TX* row = pages + (long long)slots[t] * (R + r);
@@ -169,28 +203,15 @@ __global__ __launch_bounds__(256) void latent_write_kernel(
       for (int j = threadIdx.x; j < R; j += 256)
         st(col + (long long)j * page_size, xr[j] * mult * weight[j]);
     }
-    for (int j = threadIdx.x; j < r; j += 256) {
-      float v = xr[R + j];
-      if (j < rot) {
-        const int i = j < half ? j : j - half;
-        const float c = cos_t[(long long)pos * half + i], s = sin_t[(long long)pos * half + i];
-        const float u = xr[R + i], w = xr[R + i + half];
-        v = j < half ? u * c - w * s : w * c + u * s;
-      }
-      st(row + R + j, v);
-    }
+    for (int j = threadIdx.x; j < r; j += 256)
+      st(row + R + j, turned([&](int k) { return xr[R + k]; }, j, rot, interleaved, cos_r, sin_r));
   }
+  if (!q) return;
   for (int e = threadIdx.x; e < H * r; e += 256) {
     const int h = e / r, j = e % r;
     const TX* qh = q + (long long)t * ldq + (long long)h * q_head + q_off;
-    float v = ld(qh + j);
-    if (j < rot) {
-      const int i = j < half ? j : j - half;
-      const float c = cos_t[(long long)pos * half + i], s = sin_t[(long long)pos * half + i];
-      const float u = ld(qh + i), w = ld(qh + i + half);
-      v = j < half ? u * c - w * s : w * c + u * s;
-    }
-    st(q_out + (long long)t * ldo + (long long)h * o_head + R + j, v);
+    st(q_out + (long long)t * ldo + (long long)h * o_head + R + j,
+       turned([&](int k) { return ld(qh + k); }, j, rot, interleaved, cos_r, sin_r));
   }
 }
 
@@ -198,23 +219,26 @@ RLIS_API int rlis_latent_write(const float* x, long long ldx, const float* weigh
                                int R, int r, int rot, const float* cos_t, const float* sin_t,
                                const int* positions, const int* slots, void* pages,
                                void* pages_t, int page_size, int dtype, int write, const void* q, long long ldq, int q_head, int q_off,
-                               void* q_out, long long ldo, int o_head, int H, int T,
-                               hipStream_t stream) {
+                               void* q_out, long long ldo, int o_head, int H, int T, int interleaved,
+                               const float* cq, long long ld_cq, int cq_R, const float* cq_weight,
+                               void* cq_out, hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && R > 0 && r >= 0 && rot >= 0 && rot <= r && rot % 2 == 0 && H > 0,
                "latent_write: bad sizes R=%d r=%d rot=%d", R, r, rot);
   RLIS_REQUIRE(rot == 0 || (cos_t && sin_t), "latent_write: a rotation needs its tables");
   RLIS_REQUIRE(!write || (ldx >= R + r && pages && slots && weight),
                "latent_write: the cache write needs rows, pages and slots");
   RLIS_REQUIRE(!pages_t || page_size > 0, "latent_write: the transposed copy needs the page size");
-  RLIS_REQUIRE(r == 0 || (q && q_out && q_head >= q_off + r && o_head >= R + r),
+  RLIS_REQUIRE(!q || (r > 0 && q_out && q_head >= q_off + r && o_head >= R + r),
                "latent_write: the rotated query part needs its rows");
-  if (T == 0 || (!write && r == 0)) return 0;
+  RLIS_REQUIRE(!cq || (cq_R > 0 && ld_cq >= cq_R && cq_weight && cq_out),
+               "latent_write: the queries' latent needs its rows, its weight and a result");
+  if (T == 0 || (!write && !q && !cq)) return 0;
+  const LatentQuery lq = {cq, ld_cq, cq_R, cq_weight, cq_out};
 #define LAUNCH(TX)                                                                            \
-  latent_write_kernel<TX><<<T, 256, 0, stream>>>(x, ldx, weight, eps, R, r, rot, cos_t, sin_t, \
-                                                 positions, slots, (TX*)pages, (TX*)pages_t,   \
-                                                 page_size, write,                             \
-                                                 (const TX*)q, ldq, q_head, q_off, (TX*)q_out, \
-                                                 ldo, o_head, H)
+  latent_write_kernel<TX><<<dim3(T, cq ? 2 : 1), 256, 0, stream>>>(                           \
+      x, ldx, weight, eps, R, r, rot, cos_t, sin_t, positions, slots, (TX*)pages,             \
+      (TX*)pages_t, page_size, write, (const TX*)q, ldq, q_head, q_off, (TX*)q_out, ldo,      \
+      o_head, H, interleaved, lq)
   if (dtype == RLIS_F32) LAUNCH(float);
   else if (dtype == RLIS_BF16) LAUNCH(bf16_t);
   else RLIS_REQUIRE(false, "latent_write: unknown dtype %d", dtype);

@@ -10,8 +10,10 @@
 //    front of everything (softmax scores over all experts, divided by the chosen ones' sum, are
 //    the softmax over the chosen logits alone).  A unit's bounded form: see gated_unit; units
 //    without a gate (one projection, the square of its ReLU, the down projection): plain_unit.
+//    Experts from `E` of the products on are identity experts: they have no weights, their output
+//    is the token's input itself.
 //  * moe_sort: the step's (token, choice) pairs ordered by expert, every expert's run padded to
-//    whole tiles of rows, so that a tile has one expert.  Decided on the device: nothing waits
+//    whole tiles of rows, so that a tile has one expert; pairs of identity experts take no row.  Decided on the device: nothing waits
 //    for the host.  Which row of its expert's run a pair gets does not move its result: rows of a
 //    tile do not see each other.
 //  * moe_gate_up / moe_down: the units' products on the matrix cores, tile by tile
@@ -237,7 +239,8 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   for (int i = threadIdx.x; i < max_tiles * tile_rows; i += blockDim.x) sorted[i] = -1;
   for (int i = threadIdx.x; i < max_tiles; i += blockDim.x) tile_expert[i] = -1;
   __syncthreads();
-  for (int p = threadIdx.x; p < P; p += blockDim.x) atomicAdd(&count[chosen[p]], 1);
+  for (int p = threadIdx.x; p < P; p += blockDim.x)
+    if (chosen[p] < E) atomicAdd(&count[chosen[p]], 1);
   __syncthreads();
   if (threadIdx.x == 0) {
     int tile = 0;
@@ -252,7 +255,7 @@ __global__ __launch_bounds__(1024) void moe_sort_kernel(const int* __restrict__ 
   __syncthreads();
   for (int p = threadIdx.x; p < P; p += blockDim.x) {
     const int e = chosen[p];
-    sorted[start[e] + atomicAdd(&count[e], 1)] = p;
+    if (e < E) sorted[start[e] + atomicAdd(&count[e], 1)] = p;
   }
 }
 
@@ -637,32 +640,76 @@ RLIS_API int rlis_moe_experts(const void* x, int dtype, long long ldx, const voi
 
 // ---------------------------------------------------------------------- combine
 // out[t][n] = sum over the token's `top` pairs of y[t * top + k][n], in the order of k, plus
-// addend[t][n] when there is one.
-template <typename TA>
-__global__ void moe_combine_kernel(float* __restrict__ out, const float* __restrict__ y,
-                                   const TA* __restrict__ addend, int top, int N, long long total) {
-  const long long i = (long long)blockIdx.x * blockDim.x + threadIdx.x;
+// addend[t][n] when there is one.  IDENTITY: a pair whose expert is E or above has no row in y; it
+// adds its weight times the token's input x[t][n].  V columns a thread (N a multiple of V).
+template <typename TA, typename TX, bool IDENTITY, int V>
+__global__ __launch_bounds__(256) void moe_combine_kernel(
+    float* __restrict__ out, const float* __restrict__ y, const TA* __restrict__ addend, int top,
+    int N, long long total, const int* __restrict__ chosen, const float* __restrict__ weights,
+    int E, const TX* __restrict__ x, long long ldx) {
+  const long long i = ((long long)blockIdx.x * blockDim.x + threadIdx.x) * V;
   if (i >= total) return;
   const long long t = i / N;
   const int n = (int)(i % N);
-  float s = 0.f;
-  for (int k = 0; k < top; ++k) s += y[(t * top + k) * N + n];
-  if (addend) s += ld(addend + i);
-  out[i] = s;
+  float s[V];
+#pragma unroll
+  for (int e = 0; e < V; ++e) s[e] = 0.f;
+  for (int k = 0; k < top; ++k) {
+    if (IDENTITY && chosen[t * top + k] >= E) {
+      const float w = weights[t * top + k];
+#pragma unroll
+      for (int e = 0; e < V; ++e) s[e] += w * ld(x + t * ldx + n + e);
+    } else {
+      const float* row = y + (t * top + k) * N + n;
+      if constexpr (V == 4) {
+        const float4 v = *(const float4*)row;
+        s[0] += v.x; s[1] += v.y; s[2] += v.z; s[3] += v.w;
+      } else {
+        s[0] += row[0];
+      }
+    }
+  }
+  if (addend) {
+#pragma unroll
+    for (int e = 0; e < V; ++e) s[e] += ld(addend + i + e);
+  }
+  if constexpr (V == 4) *(float4*)(out + i) = make_float4(s[0], s[1], s[2], s[3]);
+  else out[i] = s[0];
 }
 
 RLIS_API int rlis_moe_combine(float* out, const float* y, const void* addend, int addend_dtype,
-                              int T, int top, int N, hipStream_t stream) {
+                              int T, int top, int N, const int* chosen, const float* weights,
+                              int E, const void* x, int x_dtype, long long ldx,
+                              hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && top > 0 && N > 0, "moe_combine: bad sizes");
+  RLIS_REQUIRE(!x || (chosen && weights && E >= 0 && ldx >= N),
+               "moe_combine: identity experts need the choices, the weights and the inputs");
+  RLIS_REQUIRE(!x || x_dtype == RLIS_F32 || x_dtype == RLIS_BF16, "moe_combine: unknown dtype %d",
+               x_dtype);
   const long long total = (long long)T * N;
   if (total == 0) return 0;
-  const unsigned blocks = (unsigned)ceil_div_ll(total, 256);
-  if (!addend || addend_dtype == RLIS_F32)
-    moe_combine_kernel<float><<<blocks, 256, 0, stream>>>(out, y, (const float*)addend, top, N, total);
-  else if (addend_dtype == RLIS_BF16)
-    moe_combine_kernel<bf16_t><<<blocks, 256, 0, stream>>>(out, y, (const bf16_t*)addend, top, N, total);
-  else
-    RLIS_REQUIRE(false, "moe_combine: unknown dtype %d", addend_dtype);
+  const bool four = N % 4 == 0 && (uintptr_t)out % 16 == 0 && (uintptr_t)y % 16 == 0;
+  const unsigned blocks = (unsigned)ceil_div_ll(total, four ? 1024 : 256);
+#define LAUNCH(TA, TX, ID, V)                                                                   \
+  moe_combine_kernel<TA, TX, ID, V><<<blocks, 256, 0, stream>>>(                                \
+      out, y, (const TA*)addend, top, N, total, chosen, weights, E, (const TX*)x, ldx)
+#define BY_V(TA, TX, ID)                  \
+  do {                                    \
+    if (four) LAUNCH(TA, TX, ID, 4);      \
+    else LAUNCH(TA, TX, ID, 1);           \
+  } while (0)
+#define BY_X(TA)                                           \
+  do {                                                     \
+    if (!x) BY_V(TA, float, false);                        \
+    else if (x_dtype == RLIS_F32) BY_V(TA, float, true);   \
+    else BY_V(TA, bf16_t, true);                           \
+  } while (0)
+  if (!addend || addend_dtype == RLIS_F32) BY_X(float);
+  else if (addend_dtype == RLIS_BF16) BY_X(bf16_t);
+  else RLIS_REQUIRE(false, "moe_combine: unknown dtype %d", addend_dtype);
+#undef BY_X
+#undef BY_V
+#undef LAUNCH
   RLIS_LAUNCH_CHECK("moe_combine");
   return 0;
 }

@@ -10,22 +10,25 @@
 // x[t] += y[t] / sqrt(mean(y[t]^2) + eps) * weight in the float32 residual x (T, W); y is (T, W) in
 // either dtype, or `parts` float32 partial sums (part_stride elements apart) that are added in
 // order and, with round16, rounded to bfloat16 first.  The new row goes to `out` (T, W) in its
-// dtype when out is given.  y null: x stays as it is and is copied to `out`.
+// dtype when out is given, or (next_w) the norm of the new row,
+// x[t] / sqrt(mean(x[t]^2) + next_eps) * next_w, which is what a sublayer with a norm in front
+// reads.  y null: x stays as it is and is copied to `out`.
 //
 // One workgroup per token.  A thread owns up to CH chunks of four consecutive elements; all of a
 // row's loads (residual, weight, the parts eight at a time) are asked for before the sum of
 // squares is waited for, and a chunk past the row reads the row's first elements and adds
 // nothing.
-template <typename TY, typename TW, typename TO, int NT, int CH>
+template <typename TY, typename TW, typename TO, int NT, int CH, bool NEXT>
 __global__ __launch_bounds__(NT) void norm_join_kernel(
     float* __restrict__ x, const TY* __restrict__ y, int parts, long long part_stride, int round16,
-    const TW* __restrict__ weight, float eps, TO* __restrict__ out, int W) {
+    const TW* __restrict__ weight, float eps, TO* __restrict__ out, int W,
+    const TW* __restrict__ next_w, float next_eps) {
   __shared__ float red[NT / kWave];
   const long long base = (long long)blockIdx.x * W;
   int col[CH];
   bool live[CH];
   float4 xr[CH];
-  TW wt[CH][4];
+  TW wt[CH][4], nt[CH][4];
   float s[CH][4];
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
@@ -58,7 +61,10 @@ __global__ __launch_bounds__(NT) void norm_join_kernel(
       for (int c = 0; c < CH; ++c) {
         xr[c] = *(const float4*)(x + base + col[c]);
 #pragma unroll
-        for (int e = 0; e < 4; ++e) wt[c][e] = weight[col[c] + e];
+        for (int e = 0; e < 4; ++e) {
+          wt[c][e] = weight[col[c] + e];
+          if constexpr (NEXT) nt[c][e] = next_w[col[c] + e];
+        }
       }
     }
 #pragma unroll
@@ -82,6 +88,38 @@ __global__ __launch_bounds__(NT) void norm_join_kernel(
     }
   ss = block_sum<NT>(ss, red);
   const float inv = 1.0f / sqrtf(ss / (float)W + eps);
+  if constexpr (NEXT) {
+    float sn = 0.f;
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      const float xs[4] = {xr[c].x, xr[c].y, xr[c].z, xr[c].w};
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        s[c][e] = xs[e] + s[c][e] * inv * widen(wt[c][e]);
+        if (live[c]) sn += s[c][e] * s[c][e];
+      }
+      if (live[c])
+        *(float4*)(x + base + col[c]) = make_float4(s[c][0], s[c][1], s[c][2], s[c][3]);
+    }
+    sn = block_sum<NT>(sn, red);
+    const float next_inv = 1.0f / sqrtf(sn / (float)W + next_eps);
+#pragma unroll
+    for (int c = 0; c < CH; ++c) {
+      if (!live[c]) continue;
+      float r[4];
+#pragma unroll
+      for (int e = 0; e < 4; ++e) r[e] = s[c][e] * next_inv * widen(nt[c][e]);
+      if constexpr (sizeof(TO) == 2) {
+        uint2 o;
+        o.x = (uint32_t)f32_to_bf16(r[0]) | ((uint32_t)f32_to_bf16(r[1]) << 16);
+        o.y = (uint32_t)f32_to_bf16(r[2]) | ((uint32_t)f32_to_bf16(r[3]) << 16);
+        *(uint2*)(out + base + col[c]) = o;
+      } else {
+        *(float4*)(out + base + col[c]) = make_float4(r[0], r[1], r[2], r[3]);
+      }
+    }
+    return;
+  }
 #pragma unroll
   for (int c = 0; c < CH; ++c) {
     if (!live[c]) continue;
@@ -107,7 +145,8 @@ __global__ __launch_bounds__(NT) void norm_join_kernel(
 template <typename TY, typename TW, typename TO>
 __global__ __launch_bounds__(256) void norm_join_any_kernel(
     float* __restrict__ x, const TY* __restrict__ y, int parts, long long part_stride, int round16,
-    const TW* __restrict__ weight, float eps, TO* __restrict__ out, int W) {
+    const TW* __restrict__ weight, float eps, TO* __restrict__ out, int W,
+    const TW* __restrict__ next_w, float next_eps) {
   __shared__ float red[4];
   const long long base = (long long)blockIdx.x * W;
   float ss = 0.f;
@@ -117,12 +156,19 @@ __global__ __launch_bounds__(256) void norm_join_any_kernel(
   }
   ss = block_sum<256>(ss, red);
   const float inv = 1.0f / sqrtf(ss / (float)W + eps);
+  float sn = 0.f;
   for (int j = threadIdx.x; j < W; j += 256) {
     const float v = delta_sum(y + base + j, parts, part_stride, round16);
     const float r = x[base + j] + v * inv * ld(weight + j);
     x[base + j] = r;
-    if (out) st(out + base + j, r);
+    if (out && !next_w) st(out + base + j, r);
+    sn += r * r;
   }
+  if (!next_w) return;
+  // (a thread reads back the elements it has written itself)
+  const float next_inv = 1.0f / sqrtf(block_sum<256>(sn, red) / (float)W + next_eps);
+  for (int j = threadIdx.x; j < W; j += 256)
+    st(out + base + j, x[base + j] * next_inv * ld(next_w + j));
 }
 
 template <typename TO>
@@ -135,14 +181,21 @@ __global__ void cast_rows_kernel(const float* __restrict__ x, TO* __restrict__ o
 template <typename TY, typename TW, typename TO>
 static void launch_norm_join(float* x, const void* y, int parts, long long part_stride, int round16,
                              const void* w, float eps, void* out, int T, int W, bool vec,
-                             hipStream_t stream) {
-#define RLIS_JOIN(NT, CH)                                                                         \
-  norm_join_kernel<TY, TW, TO, NT, CH><<<T, NT, 0, stream>>>(x, (const TY*)y, parts, part_stride, \
-                                                             round16, (const TW*)w, eps, (TO*)out, W)
+                             const void* next_w, float next_eps, hipStream_t stream) {
+#define RLIS_JOIN_AS(NT, CH, NEXT)                                                             \
+  norm_join_kernel<TY, TW, TO, NT, CH, NEXT><<<T, NT, 0, stream>>>(                            \
+      x, (const TY*)y, parts, part_stride, round16, (const TW*)w, eps, (TO*)out, W,            \
+      (const TW*)next_w, next_eps)
+#define RLIS_JOIN(NT, CH)                            \
+  do {                                               \
+    if (next_w) RLIS_JOIN_AS(NT, CH, true);          \
+    else RLIS_JOIN_AS(NT, CH, false);                \
+  } while (0)
   const int quads = W / 4;
   if (!vec || quads > 4096)
     norm_join_any_kernel<TY, TW, TO><<<T, 256, 0, stream>>>(x, (const TY*)y, parts, part_stride,
-                                                            round16, (const TW*)w, eps, (TO*)out, W);
+                                                            round16, (const TW*)w, eps, (TO*)out, W,
+                                                            (const TW*)next_w, next_eps);
   else if (quads <= 64) RLIS_JOIN(64, 1);
   else if (quads <= 128) RLIS_JOIN(128, 1);
   else if (quads <= 256) RLIS_JOIN(256, 1);
@@ -152,12 +205,15 @@ static void launch_norm_join(float* x, const void* y, int parts, long long part_
   else if (quads <= 2048) RLIS_JOIN(1024, 2);
   else RLIS_JOIN(1024, 4);
 #undef RLIS_JOIN
+#undef RLIS_JOIN_AS
 }
 
 RLIS_API int rlis_norm_join(float* x, const void* y, int y_dtype, int parts, long long part_stride,
                             int round16, const void* weight, int w_dtype, float eps, void* out,
-                            int out_dtype, int T, int W, hipStream_t stream) {
+                            int out_dtype, int T, int W, const void* next_w, float next_eps,
+                            hipStream_t stream) {
   RLIS_REQUIRE(T >= 0 && W > 0, "norm_join: bad sizes T=%d W=%d", T, W);
+  RLIS_REQUIRE(!next_w || (y && out), "norm_join: a norm behind the join needs a row and a result");
   RLIS_REQUIRE(y == nullptr || (weight && parts >= 1), "norm_join: a row to join needs a weight");
   RLIS_REQUIRE(parts == 1 || (y_dtype == RLIS_F32 && part_stride >= (long long)T * W),
                "norm_join: a stack of partial sums is float32 and whole");
@@ -182,10 +238,10 @@ RLIS_API int rlis_norm_join(float* x, const void* y, int y_dtype, int parts, lon
   do {                                                                                           \
     if (out && out_dtype == RLIS_F32)                                                            \
       launch_norm_join<TY, TW, float>(x, y, parts, part_stride, round16, weight, eps, out, T, W, \
-                                      vec, stream);                                              \
+                                      vec, next_w, next_eps, stream);                            \
     else                                                                                         \
       launch_norm_join<TY, TW, bf16_t>(x, y, parts, part_stride, round16, weight, eps, out, T, W, \
-                                       vec, stream);                                             \
+                                       vec, next_w, next_eps, stream);                           \
   } while (0)
   if (y_dtype == RLIS_F32 && w_dtype == RLIS_F32) RLIS_BY_OUT(float, float);
   else if (y_dtype == RLIS_F32) RLIS_BY_OUT(float, bf16_t);

@@ -4,8 +4,9 @@ from .gipotar import gipotar_spec
 from .lagedra import lagedra_spec
 from .llama import llama_spec
 from .pamolix import pamolix_spec
+from .pozelix import pozelix_spec
 from .ralitar import ralitar_spec
-from .spec import LayerSpec, Model, ModelSpec, RunEntry
+from .spec import JunctionSpec, LayerSpec, Model, ModelSpec, RunEntry
 
-__all__ = ["LayerSpec", "Model", "ModelSpec", "RunEntry", "bekunex_spec", "gipotar_spec",
-           "lagedra_spec", "llama_spec", "pamolix_spec", "ralitar_spec"]
+__all__ = ["JunctionSpec", "LayerSpec", "Model", "ModelSpec", "RunEntry", "bekunex_spec", "gipotar_spec",
+           "lagedra_spec", "llama_spec", "pamolix_spec", "pozelix_spec", "ralitar_spec"]

@@ -2,8 +2,9 @@
 
 ``ModelSpec`` lists the layers (each a block specification with its weight-name prefix) and
 the *run order*: a list of ``RunEntry`` that names which layer runs when.  A layer may be
-named more than once (each run then has a cache of its own), and a run may read the cache
-another run writes (``cache_of``) instead of writing its own.  ``Model`` builds the parts
+named more than once (each run then has a cache of its own), a run may read the cache
+another run writes (``cache_of``) instead of writing its own, and a run may have a junction in
+front of it (``junction``: something that happens to the residual stream there).  ``Model`` builds the parts
 through the registries, groups the cache requests of the runs into page groups, and runs a
 step: embedding, the run order, final norm on the wanted rows, head."""
 from __future__ import annotations
@@ -13,7 +14,7 @@ from typing import Any, Dict, List, Optional, Tuple
 
 import torch
 
-from ..parts.base import (Block, BuildContext, CacheRequest, PartSpec,
+from ..parts.base import (Block, BuildContext, CacheRequest, Junction, PartSpec,
                           ResidualStream, TensorSpec, create, normed, tensor_specs)
 
 
@@ -28,6 +29,15 @@ class RunEntry:
     layer: int
     # Index into the run order of the run whose cache this run reads; None: a cache of its own.
     cache_of: Optional[int] = None
+    # Index into the specification's junctions: what happens to the stream right in front of
+    # this run; None: nothing.
+    junction: Optional[int] = None
+
+
+@dataclass
+class JunctionSpec:
+    part: PartSpec
+    prefix: str
 
 
 @dataclass
@@ -44,6 +54,7 @@ class ModelSpec:
     run_order: Optional[List[RunEntry]] = None     # None: every layer once, in order
     # Checkpoint tensors that may be present without being read.
     optional_tensors: Tuple[str, ...] = ()
+    junctions: List[JunctionSpec] = field(default_factory=list)
 
     def runs(self) -> List[RunEntry]:
         if self.run_order is not None:
@@ -54,6 +65,8 @@ class ModelSpec:
         out = tensor_specs("embedding", self.embedding, self.embedding_prefix)
         for layer in self.layers:
             out += tensor_specs("block", layer.block, layer.prefix)
+        for j in self.junctions:
+            out += tensor_specs("junction", j.part, j.prefix)
         out += tensor_specs("norm", self.final_norm, self.final_norm_prefix)
         out += tensor_specs("head", self.head, self.head_prefix)
         seen, unique = set(), []
@@ -68,6 +81,9 @@ class ModelSpec:
         for i, r in enumerate(runs):
             if not 0 <= r.layer < len(self.layers):
                 raise ValueError(f"run {i} names layer {r.layer}, the model has {len(self.layers)}")
+            if r.junction is not None and not 0 <= r.junction < len(self.junctions):
+                raise ValueError(f"run {i} names junction {r.junction}, the model has "
+                                 f"{len(self.junctions)}")
             if r.cache_of is not None:
                 if not 0 <= r.cache_of < i:
                     raise ValueError(f"run {i} reads the cache of run {r.cache_of}, which does "
@@ -108,11 +124,14 @@ class Model:
                            max_positions=max_positions)
         self.embedding = create("embedding", spec.embedding, spec.embedding_prefix, ctx)
         self.layers: List[Block] = [create("block", l.block, l.prefix, ctx) for l in spec.layers]
+        self.junctions: List[Junction] = [create("junction", j.part, j.prefix, ctx)
+                                          for j in spec.junctions]
         self.final_norm = create("norm", spec.final_norm, spec.final_norm_prefix, ctx)
         self.head = create("head", spec.head, spec.head_prefix, ctx)
         self.runs = spec.runs()
         self.graph_safe = all(getattr(p, "graph_safe", False)
-                              for p in (self.embedding, *self.layers, self.final_norm, self.head))
+                              for p in (self.embedding, *self.layers, *self.junctions,
+                                        self.final_norm, self.head))
         self._plan_cache()
         if device.type == "cuda":
             # the library's products are tried out over the weights of one shape in turn
@@ -131,7 +150,8 @@ class Model:
         """Every tensor that a part of the model holds as an attribute (parts within parts
         included)."""
         from ..parts.base import Part
-        todo, seen = [self.embedding, *self.layers, self.final_norm, self.head], set()
+        todo, seen = [self.embedding, *self.layers, *self.junctions, self.final_norm,
+                      self.head], set()
         while todo:
             part = todo.pop()
             if id(part) in seen:
@@ -194,7 +214,10 @@ class Model:
         else:
             x = self.embedding.forward(step.ids, step.positions)
         stream = ResidualStream(x, self.act_dtype)
+        kept = [j.begin(stream) for j in self.junctions]
         for i, run in enumerate(self.runs):
+            if run.junction is not None:
+                self.junctions[run.junction].forward(stream, kept[run.junction])
             self.layers[run.layer].forward(stream, step, pools.binding(self.bindings[i]))
         if step.num_logit_rows == 0:
             return torch.empty((0, self.spec.vocab_size), dtype=torch.float32, device=self.device)

@@ -490,17 +490,27 @@ def geglu(gu: torch.Tensor) -> torch.Tensor:
 
 
 def norm_join(resid: torch.Tensor, y: Optional[torch.Tensor], weight: Optional[torch.Tensor],
-              eps: float, out_dtype: Optional[torch.dtype] = None, round_parts: bool = False
+              eps: float, out_dtype: Optional[torch.dtype] = None, round_parts: bool = False,
+              next_weight: Optional[torch.Tensor] = None, next_eps: float = 0.0
               ) -> Optional[torch.Tensor]:
     """``resid += y / sqrt(mean(y^2) + eps) * weight`` row by row in the float32 residual
     ``(T, W)``; ``y`` is ``(T, W)``, or a stack ``(S, T, W)`` of float32 partial sums that are added in
     order and with ``round_parts`` rounded to bfloat16 first.  Returns the new residual in
     ``out_dtype`` (the residual itself for float32, None for None).  ``y`` None: the residual
-    stays as it is."""
+    stays as it is.  ``next_weight`` (of ``weight``'s dtype): what comes back, in ``out_dtype``, is
+    the norm of the new residual, ``resid / sqrt(mean(resid^2) + next_eps) * next_weight``."""
     _check(resid, "residual", torch.float32, 2)
     if not resid.is_contiguous():
         raise KernelError("norm_join: residual must be contiguous")
     T, W = resid.shape
+    next_ptr = None
+    if next_weight is not None:
+        _check(next_weight, "next norm weight", ndim=1)
+        if y is None or out_dtype is None or next_weight.dtype != weight.dtype \
+                or next_weight.numel() != W or not next_weight.is_contiguous():
+            raise KernelError("norm_join: a norm behind the join takes a row that joins, a result "
+                              "dtype and a weight of the first norm's dtype and size")
+        next_ptr = next_weight.data_ptr()
     if y is None:
         if out_dtype in (None, torch.float32):
             return None if out_dtype is None else resid
@@ -512,12 +522,14 @@ def norm_join(resid: torch.Tensor, y: Optional[torch.Tensor], weight: Optional[t
             raise KernelError(f"norm_join: weight has {weight.numel()} entries, rows have {W}")
         y_args, w_args = (y.data_ptr(), _dt(y)), (weight.data_ptr(), _dt(weight))
     out = None
-    if out_dtype == torch.bfloat16:
-        out = torch.empty((T, W), dtype=torch.bfloat16, device=resid.device)
+    if out_dtype == torch.bfloat16 or next_ptr is not None:
+        out = torch.empty((T, W), dtype=out_dtype, device=resid.device)
     lib.call("rlis_norm_join", resid.data_ptr(), *y_args, parts, T * W,
              int(bool(round_parts) and y is not None and y.dim() > 2), *w_args, float(eps),
-             None if out is None else out.data_ptr(), _DT[torch.bfloat16], T, W, lib.stream_ptr())
-    return resid if out_dtype == torch.float32 else out
+             None if out is None else out.data_ptr(),
+             _DT[torch.bfloat16 if out is None else out.dtype], T, W, next_ptr, float(next_eps),
+             lib.stream_ptr())
+    return resid if out is None and out_dtype == torch.float32 else out
 
 
 def side_gate_(z: torch.Tensor, table: torch.Tensor, column: int, ids: torch.Tensor
@@ -1082,6 +1094,45 @@ def rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim
              nh, nkv, d, rot, cos_ptr, sin_ptr, _i32(positions, "positions", T), sp, kp, vp,
              page_size, int(bool(write_kv)), int(bool(interleaved)), int(bool(rotate_q)),
              lib.stream_ptr())
+
+
+def norm_rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
+                       real_dim: int, eps: float, cos: Optional[torch.Tensor],
+                       sin: Optional[torch.Tensor], positions: torch.Tensor,
+                       slots: Optional[torch.Tensor], k_pages: Optional[torch.Tensor],
+                       v_pages: Optional[torch.Tensor], page_size: int, write_kv: bool = True,
+                       interleaved: bool = False) -> None:
+    """``rope_kv_write`` for queries and keys that are divided by their root mean square behind
+    the rotation: every q and k head of ``qkv (T, (nh + 2 nkv) d)`` is rotated and then divided by
+    ``sqrt(mean(head^2) + eps)``, the mean over its first ``real_dim`` numbers (the others are
+    zero padding).  q in place; with ``write_kv`` k and v go to the pages."""
+    stride = _rows_contig(qkv, "qkv")
+    T, nh, nkv, d = qkv.shape[0], int(num_heads), int(num_kv_heads), int(head_dim)
+    if qkv.shape[1] != (nh + 2 * nkv) * d:
+        raise KernelError(f"norm_rope_kv_write: qkv has {qkv.shape[1]} columns, expected "
+                          f"{(nh + 2 * nkv) * d}")
+    rot, cos_ptr, sin_ptr = 0, None, None
+    if cos is not None:
+        for t in (cos, sin):
+            _check(t, "norm_rope_kv_write angles", torch.float32, 2)
+        if cos.shape != sin.shape or not (cos.is_contiguous() and sin.is_contiguous()):
+            raise KernelError("norm_rope_kv_write: cos and sin must match and be contiguous")
+        rot, cos_ptr, sin_ptr = 2 * cos.shape[1], cos.data_ptr(), sin.data_ptr()
+    kp = vp = sp = None
+    if write_kv:
+        if k_pages is None or v_pages is None or slots is None:
+            raise KernelError("norm_rope_kv_write: a cache write needs pages and slots")
+        for t, name, shape in ((k_pages, "k_pages", (nkv, page_size, d)),
+                               (v_pages, "v_pages", (nkv, d, page_size))):
+            _check(t, name, qkv.dtype, 4)
+            if tuple(t.shape[1:]) != shape or not t.is_contiguous():
+                raise KernelError(f"norm_rope_kv_write: {name} has shape {tuple(t.shape)}, expected "
+                                  f"(pages, {shape[0]}, {shape[1]}, {shape[2]}) contiguous")
+        kp, vp, sp = k_pages.data_ptr(), v_pages.data_ptr(), _i32(slots, "slots", T)
+    lib.call("rlis_norm_rope_kv_write", qkv.data_ptr(), _dt(qkv), stride, nh * d, (nh + nkv) * d, T,
+             nh, nkv, d, int(real_dim), rot, float(eps), cos_ptr, sin_ptr,
+             _i32(positions, "positions", T), sp, kp, vp, page_size, int(bool(interleaved)),
+             int(bool(write_kv)), lib.stream_ptr())
 
 
 def copy_pages(pages: torch.Tensor, src: torch.Tensor, dst: torch.Tensor) -> None:

@@ -61,16 +61,19 @@ def latent_write(x: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps:
                  sin: Optional[torch.Tensor], positions: torch.Tensor,
                  slots: Optional[torch.Tensor], pages: Optional[torch.Tensor],
                  q: Optional[torch.Tensor], q_head: int, q_out: Optional[torch.Tensor],
-                 heads: int, pages_t: Optional[torch.Tensor] = None) -> None:
+                 heads: int, pages_t: Optional[torch.Tensor] = None, interleaved: bool = False,
+                 query_latent: Optional[tuple] = None) -> None:
     """For every token of the step: the first ``rank`` columns of ``x`` (float32), divided by
     their root mean square (``eps`` inside the root) and multiplied by ``weight``, go to the
     token's row of ``pages (pages, page size, rank + rot_width)`` at ``slots``; the
     ``rot_width`` columns behind them follow, the first ``rot_dims`` of them rotated by the
-    token's position (entry i with entry i + rot_dims / 2, angles from the float32 tables
-    ``cos``/``sin (positions, rot_dims / 2)``).  The last ``rot_width`` numbers of every head
+    token's position (entry i with entry i + rot_dims / 2, or with ``interleaved`` entry 2i with
+    2i + 1, angles from the float32 tables ``cos``/``sin (positions, rot_dims / 2)``).  The last ``rot_width`` numbers of every head
     of ``q`` (heads ``q_head`` apart) are rotated the same way into ``q_out`` behind each
     head's first ``rank`` columns (heads ``rank + rot_width`` apart).  ``x`` None: nothing is
-    written to the cache (a mixer that reads another's).  ``pages_t (pages, rank, page size)``:
+    written to the cache (a mixer that reads another's); ``q`` None: no queries are rotated.
+    ``query_latent = (cq, weight, out)``: the rows of ``cq (T, Rq)`` float32 go through the same
+    norm with a weight of their own to ``out (T, Rq)`` contiguous, of the pages' dtype.  ``pages_t (pages, rank, page size)``:
     the latent is stored there once more, with the positions of a page innermost (what the
     matrix-core attention kernel reads as values)."""
     T = positions.numel() if q is None else q.shape[0]
@@ -95,17 +98,29 @@ def latent_write(x: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps:
                               "(pages, rank, page size) of the pages' dtype")
     ldq = ldo = 0
     dtype = pages.dtype if pages is not None else (q.dtype if q is not None else torch.float32)
-    if rot_width:
+    if rot_width and q is None and x is None:
+        raise KernelError("latent_write: neither rows for the cache nor queries to rotate")
+    if rot_width and q is not None:
         ldq, ldo = _rows2(q, "latent_write q"), _rows2(q_out, "latent_write q_out")
         if q.dtype != dtype or q_out.dtype != dtype or q_head < rot_width \
                 or q.shape[1] < heads * q_head or q_out.shape[1] < heads * D:
             raise KernelError("latent_write: the queries' rows do not match the heads")
-        if rot_dims:
-            for t in (cos, sin):
-                if t is None or t.dtype != torch.float32 or not t.is_contiguous() \
-                        or t.shape[1] != rot_dims // 2:
-                    raise KernelError("latent_write: the rotation needs float32 tables "
-                                      "(positions, rot_dims / 2)")
+    if rot_width and rot_dims:
+        for t in (cos, sin):
+            if t is None or t.dtype != torch.float32 or not t.is_contiguous() \
+                    or t.shape[1] != rot_dims // 2:
+                raise KernelError("latent_write: the rotation needs float32 tables "
+                                  "(positions, rot_dims / 2)")
+    cq_args = (None, 0, 0, None, None)
+    if query_latent is not None:
+        cq, cq_w, cq_out = query_latent
+        ld_cq = _rows2(cq, "latent_write cq")
+        if cq.dtype != torch.float32 or cq.shape[0] != T or cq_w.dtype != torch.float32 \
+                or cq_w.numel() != cq.shape[1] or not cq_w.is_contiguous() \
+                or cq_out.shape != cq.shape or cq_out.dtype != dtype or not cq_out.is_contiguous():
+            raise KernelError("latent_write: the queries' latent must be float32 (T, Rq) with a "
+                              "float32 weight and a contiguous result of the pages' dtype")
+        cq_args = (cq.data_ptr(), ld_cq, cq.shape[1], cq_w.data_ptr(), cq_out.data_ptr())
     lib.call("rlis_latent_write", None if not write else x.data_ptr(), ldx,
              None if not write else weight.data_ptr(), float(eps), int(rank), int(rot_width),
              int(rot_dims), None if cos is None else cos.data_ptr(),
@@ -115,7 +130,8 @@ def latent_write(x: Optional[torch.Tensor], weight: Optional[torch.Tensor], eps:
              None if pages_t is None or not write else pages_t.data_ptr(),
              0 if pages is None else pages.shape[1], _DT[dtype], int(write),
              None if q is None else q.data_ptr(), ldq, int(q_head), int(q_head - rot_width),
-             None if q_out is None else q_out.data_ptr(), ldo, D, int(heads), T, lib.stream_ptr())
+             None if q is None else q_out.data_ptr(), ldo, D, int(heads), T,
+             int(bool(interleaved)), *cq_args, lib.stream_ptr())
 
 
 # "matrix": bfloat16 attention over cached latents runs on the matrix cores where it applies;

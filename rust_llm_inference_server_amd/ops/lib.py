@@ -30,7 +30,7 @@ _SIGNATURES = {
     "rlis_add_rmsnorm": [P, P, I, P, I, P, I, P, I, I, F, I, I, L, I, F, P],
     "rlis_swiglu": [P, P, I, I, I, P],
     "rlis_geglu": [P, P, I, I, I, P],
-    "rlis_norm_join": [P, P, I, I, L, I, P, I, F, P, I, I, I, P],
+    "rlis_norm_join": [P, P, I, I, L, I, P, I, F, P, I, I, I, P, F, P],
     "rlis_side_gate": [P, I, L, P, L, P, I, I, P],
     "rlis_embed_pairs": [P, P, P, I, P, I, I, I, F, L, L, P, L, P, P, P, P],
     "rlis_row_prepare": [P, P, I, L, I, I, I, I, I, P, P, P, F, P, P, I, P, I, P],
@@ -49,7 +49,8 @@ _SIGNATURES = {
     "rlis_add_layernorm": [P, P, I, P, P, I, P, I, P, I, I, F, I, I, L, I, F, P],
     "rlis_scale": [P, I, L, F, P],
     "rlis_head_linear": [P, I, L, I, P, P, I, L, I, I, I, I, I, P],
-    "rlis_latent_write": [P, L, P, F, I, I, I, P, P, P, P, P, P, I, I, I, P, L, I, I, P, L, I, I, I, P],
+    "rlis_latent_write": [P, L, P, F, I, I, I, P, P, P, P, P, P, I, I, I, P, L, I, I, P, L, I, I, I, I,
+                          P, L, I, P, P, P],
     "rlis_latent_attention_mfma": [P, L, P, L, P, P, P, I, P, P, I, I, I, I, I, I, F, I, P, I, I, P],
     "rlis_latent_attention": [P, I, L, P, L, P, P, I, P, P, I, I, I, I, I, F, I, P, P],
     "rlis_sigmoid_gate": [P, L, P, L, I, I, I, P],
@@ -57,11 +58,12 @@ _SIGNATURES = {
     "rlis_moe_route": [P, L, P, I, I, I, I, I, F, P, P, I, I, I, P, P],
     "rlis_moe_sort": [P, I, I, I, I, P, P, P],
     "rlis_moe_experts": [P, I, L, P, P, P, P, P, I, I, I, I, I, P, P, F, F, P],
-    "rlis_moe_combine": [P, P, P, I, I, I, I, P],
+    "rlis_moe_combine": [P, P, P, I, I, I, I, P, P, I, P, I, L, P],
     "rlis_delta_scan": [P, L, P, P, P, L, P, P, L, P, P, P, L, P, P, I, I, I, I, I, I, P],
     "rlis_decay_scan": [P, P, P, P, P, L, P, P, P, L, P, P, I, I, I, I, P],
     "rlis_head_norm_gate": [P, I, P, P, I, P, I, L, I, I, I, F, I, P],
     "rlis_rope_kv_write": [P, I, L, I, I, I, I, I, I, I, P, P, P, P, P, P, I, I, I, I, P],
+    "rlis_norm_rope_kv_write": [P, I, L, I, I, I, I, I, I, I, I, F, P, P, P, P, P, P, I, I, I, P],
     "rlis_copy_pages": [P, I, I, L, L, P, P, I, P],
     "rlis_gemm_plain": [P, I, P, I, P, I, I, I, I, L, L, L, P],
     "rlis_gemm_bf16_mfma": [P, P, P, I, I, I, I, L, L, L, P],

@@ -86,7 +86,7 @@ def route(logits: torch.Tensor, correction: Optional[torch.Tensor], groups: int,
 def routed_units(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
                  chosen: torch.Tensor, weights: torch.Tensor,
                  addend: Optional[torch.Tensor] = None, limit: float = 0.0,
-                 alpha: float = 1.0, plain: bool = False) -> torch.Tensor:
+                 alpha: float = 1.0, plain: bool = False, identity: bool = False) -> torch.Tensor:
     """``out[t] = sum_k weights[t, k] * unit(chosen[t, k], x[t])  (+ addend[t])`` in float32,
     where unit ``e`` is ``Wd[e] (silu(Wg[e] x) * (Wu[e] x))`` with ``w_gate_up (E, 2 F, W)``
     (an expert's gate rows in front of its up rows) and ``w_down (E, W, F)``, both in the dtype
@@ -94,7 +94,8 @@ def routed_units(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
     units are of the bounded kind, ``Wd[e] (g sigmoid(alpha g) (u + 1))`` with
     ``g = min(Wg[e] x, limit)`` and ``u = clamp(Wu[e] x, -limit, limit)``.  ``plain``: the units
     are not gated, ``Wd[e] relu(Wu[e] x)^2`` with ``w_gate_up (E, F, W)`` the one projection
-    ``Wu`` (an even number of rows) and ``w_down (E, W, F)``."""
+    ``Wu`` (an even number of rows) and ``w_down (E, W, F)``.  ``identity``: a choice of E or above
+    stands for a unit without weights whose output is ``x[t]`` itself."""
     if not x.is_cuda or x.dim() != 2 or x.dtype not in _DT or (x.shape[1] > 1 and x.stride(1) != 1):
         raise KernelError("routed_units: x must be (T, W) on the GPU with contiguous rows")
     T, W = x.shape
@@ -135,5 +136,7 @@ def routed_units(x: torch.Tensor, w_gate_up: torch.Tensor, w_down: torch.Tensor,
         raise KernelError("routed_units: the addend must be a contiguous (T, W) tensor")
     lib.call("rlis_moe_combine", out.data_ptr(), y.data_ptr(),
              None if addend is None else addend.data_ptr(),
-             0 if addend is None else _DT[addend.dtype], T, top, W, lib.stream_ptr())
+             0 if addend is None else _DT[addend.dtype], T, top, W, chosen.data_ptr(),
+             weights.data_ptr(), E, x.data_ptr() if identity else None, _DT[x.dtype], ldx,
+             lib.stream_ptr())
     return out

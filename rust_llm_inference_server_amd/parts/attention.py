@@ -60,6 +60,9 @@ class PagedAttention(Mixer):
       projection (with its bias) gives them, in front of norm and rotation.
     * ``qk_norm`` with ``"whole": True``: the norm runs over a token's whole row of queries (and
       of keys) at once, in front of the cut into heads; the weights have the row's size.
+    * ``qk_norm`` of ``{"eps": e, "behind_rotation": True}``: every query and key head is divided
+      by the root mean square of its own numbers behind the rotation, without a weight; one
+      kernel rotates, norms and writes the cache.
     * ``channel_gate``: the name of a projection ``(num_heads * value_dim, hidden_size)`` of the
       mixer's input; its sigmoid multiplies the concatenated heads element by element, in front
       of the output projection.
@@ -112,7 +115,7 @@ class PagedAttention(Mixer):
                     (("q", nh * d), ("k", nkv * d), ("v", nkv * dv))
                     if c == "q" or (own_v if c == "v" else own_kv)]
         norm = params.get("qk_norm")
-        if norm:
+        if norm and not norm.get("behind_rotation"):
             size = {"q": nh * d, "k": nkv * d} if norm.get("whole") else {"q": d, "k": d}
             out += [TensorSpec(join(prefix, norm[c]), (size[c],), init="ones_normal", std=0.1)
                     for c in "qk" if c == "q" or own_kv]
@@ -170,6 +173,11 @@ class PagedAttention(Mixer):
         self.keys_as_values = bool(params.get("keys_as_values"))
         norm = params.get("qk_norm") or {}
         self.whole_norm = bool(norm.get("whole"))
+        self.turned_norm = bool(norm.get("behind_rotation"))
+        if self.turned_norm and (self.whole_norm or self.shared_kv or self.keys_as_values
+                                 or params.get("query_temperature")):
+            raise ValueError("attention: the norm behind the rotation is built for layers with "
+                             "keys and values of their own and no temperature")
         # the layer's rows are laid out (and rotated) by one kernel in front of the attention
         self.prepared = self.keys_as_values or self.whole_norm
         if self.chunk is not None and (self.window or params.get("keep_first")):
@@ -228,6 +236,7 @@ class PagedAttention(Mixer):
         self.norm_eps = 0.0
         if norm:
             self.norm_eps = float(norm["eps"])
+        if norm and not self.turned_norm:
             self.q_norm = ctx.take(join(prefix, norm["q"])).to(torch.float32).contiguous()
             if not self.shared_kv:
                 self.k_norm = ctx.take(join(prefix, norm["k"])).to(torch.float32).contiguous()
@@ -366,23 +375,48 @@ class PagedAttention(Mixer):
             return self._forward_prepared(x, step, binding, group)
         rows = self._project(x, step, binding)
         qkv = rows[:, :self.qkv_cols] if self.gated else rows
-        out = ops.rope_attention(qkv, self.num_heads, self.num_kv_heads, self.head_dim,
-                                 self.position.cos, self.position.sin, step.positions,
-                                 group.slots, binding.k_pages, binding.v_pages, group.page_size,
-                                 group.block_tables, step, self.scale, self.window,
-                                 write_kv=binding.writes and not self.shared_kv,
-                                 plan=step.plans.get(self.planner.key()),
-                                 interleaved=bool(getattr(self.position, "interleaved", False)),
-                                 bias_slopes=getattr(self.position, "bias_slopes", None),
-                                 counters=binding.counters, head_scales=self.head_scales,
-                                 softcap=self.softcap, sinks=self.sinks,
-                                 keep_first=self.keep_first, chunk=self.chunk)
+        if self.turned_norm:
+            out = self._attend_normed(qkv, step, binding, group)
+        else:
+            out = self._attend(qkv, step, binding, group)
         if self.channel_gated:
             at = self.gate_at
             ops.sigmoid_gate_(out, rows[:, at:at + out.shape[1]])
         elif self.gated:
             ops.head_gate_(out, rows[:, self.qkv_cols:], self.num_heads, self.head_dim)
         return ops.pending_linear(out, self.w_o, self.act_dtype)
+
+    def _attend_normed(self, qkv: torch.Tensor, step: Any, binding: CacheBinding, group: Any
+                       ) -> torch.Tensor:
+        """Queries and keys normed behind their rotation: one kernel in front of the attention."""
+        pos = self.position
+        ops.norm_rope_kv_write(qkv, self.num_heads, self.num_kv_heads, self.head_dim, self.qk_dim,
+                               self.norm_eps, pos.cos, pos.sin, step.positions, group.slots,
+                               binding.k_pages, binding.v_pages, group.page_size,
+                               write_kv=binding.writes,
+                               interleaved=bool(getattr(pos, "interleaved", False)))
+        return ops.paged_attention(qkv, self.num_heads, self.num_kv_heads, self.head_dim,
+                                   binding.k_pages, binding.v_pages, group.page_size,
+                                   group.block_tables, step, self.scale, self.window,
+                                   plan=step.plans.get(self.planner.key()),
+                                   bias_slopes=getattr(pos, "bias_slopes", None),
+                                   counters=binding.counters, head_scales=self.head_scales,
+                                   softcap=self.softcap, sinks=self.sinks,
+                                   keep_first=self.keep_first, chunk=self.chunk)
+
+    def _attend(self, qkv: torch.Tensor, step: Any, binding: CacheBinding, group: Any
+                ) -> torch.Tensor:
+        return ops.rope_attention(qkv, self.num_heads, self.num_kv_heads, self.head_dim,
+                                  self.position.cos, self.position.sin, step.positions,
+                                  group.slots, binding.k_pages, binding.v_pages, group.page_size,
+                                  group.block_tables, step, self.scale, self.window,
+                                  write_kv=binding.writes and not self.shared_kv,
+                                  plan=step.plans.get(self.planner.key()),
+                                  interleaved=bool(getattr(self.position, "interleaved", False)),
+                                  bias_slopes=getattr(self.position, "bias_slopes", None),
+                                  counters=binding.counters, head_scales=self.head_scales,
+                                  softcap=self.softcap, sinks=self.sinks,
+                                  keep_first=self.keep_first, chunk=self.chunk)
 
     def _forward_prepared(self, x: Any, step: Any, binding: CacheBinding, group: Any) -> Any:
         """Layers whose keys serve as values behind norms over whole rows: one kernel adds the

@@ -170,7 +170,7 @@ class BuildContext:
 # ---------------------------------------------------------------------- registries
 _REGISTRIES: Dict[str, Dict[str, Type["Part"]]] = {
     "mixer": {}, "feed_forward": {}, "norm": {}, "position": {}, "block": {},
-    "embedding": {}, "head": {},
+    "embedding": {}, "head": {}, "junction": {},
 }
 
 
@@ -354,6 +354,19 @@ class Block(Part):
         raise NotImplementedError
 
 
+class Junction(Part):
+    """Something that happens to the residual stream between two layer runs.  ``begin(stream)``
+    is called once a step, on the embedding output in front of the first layer, and keeps what
+    the part wants of it for the step; ``forward(stream, kept)`` gets that back wherever the run
+    order names the part."""
+
+    def begin(self, stream: "ResidualStream") -> Any:
+        return None
+
+    def forward(self, stream: "ResidualStream", kept: Any) -> None:
+        raise NotImplementedError
+
+
 class Embedding(Part):
     # True when forward also takes the step and the part's binding (``forward(ids, positions,
     # step=..., binding=...)``): a part that looks at earlier tokens or keeps state per request.
@@ -505,8 +518,7 @@ class ResidualStream:
         if norm is None:
             self.flush()
             return ops.norm_join(self.x, None, None, 0.0, self.act_dtype)
-        delta, self.pending = self.delta(), None
-        return norm.join(self, delta, self.act_dtype)
+        return norm.join(self, self.take_raw(), self.act_dtype)
 
     def take_delta(self) -> Tuple[Optional[torch.Tensor], float]:
         """The pending delta as a tensor with its multiplier; the stream then has none."""
@@ -515,6 +527,13 @@ class ResidualStream:
         delta, scale = self.delta(), self.pending_scale
         self.pending, self.pending_scale = None, 1.0
         return delta, scale
+
+    def take_raw(self) -> torch.Tensor:
+        """The pending delta as a tensor, in front of the norm it is to pass (the caller applies
+        that); the stream then has none."""
+        self.pending_norm = None
+        delta, self.pending = self.delta(), None
+        return delta
 
     def delta(self) -> Optional[torch.Tensor]:
         """The pending delta as a tensor (a product that has not run yet runs now)."""
@@ -527,9 +546,8 @@ class ResidualStream:
     def flush(self) -> torch.Tensor:
         """Fold a pending delta into the residual and return the residual."""
         if self.pending is not None and self.pending_norm is not None:
-            norm, self.pending_norm = self.pending_norm, None
-            delta, self.pending = self.delta(), None
-            norm.join(self, delta, None)
+            norm = self.pending_norm
+            norm.join(self, self.take_raw(), None)
         if self.pending is not None:
             from .. import ops
             ops.add_residual(self.x, self.delta(), round_parts=self.round_parts,

@@ -1,6 +1,7 @@
 """Decoder blocks.  The pre-norm block: ``x += mixer(norm(x)); x += feed_forward(norm(x))``
 (crates/model/src/llama.rs:264-271).  The post-norm block: ``x += norm(mixer(x)); x +=
-norm(feed_forward(x))``.  Which mixer, feed-forward and norms it holds, and under
+norm(feed_forward(x))``.  The sandwich block has norms in front and behind: ``x +=
+post(mixer(norm(x)))`` and so on.  Which mixer, feed-forward and norms it holds, and under
 which weight names, is given by its parameters, layer by layer.  The parallel block:
 ``x += mixer(h) + feed_forward(h)`` with ``h = norm(x)``, one norm that both sublayers read, or
 ``x += mixer(norm(x)) + feed_forward(ffn_norm(x))`` with a norm each of the same x.  Behind
@@ -45,9 +46,12 @@ class PreNormBlock(Block):
         super().__init__(params, prefix, ctx)
         built = {slot: create(category, params[slot], join(prefix, params["names"][slot]), ctx)
                  for slot, category in self._slots(params)}
+        self._take(built)
+        self.residual_scale = float(params.get("residual_scale", 1.0))
+
+    def _take(self, built: Dict[str, Any]) -> None:
         self.mixer_norm, self.mixer = built["mixer_norm"], built["mixer"]
         self.ffn_norm, self.feed_forward = built.get("ffn_norm"), built.get("feed_forward")
-        self.residual_scale = float(params.get("residual_scale", 1.0))
 
     @property
     def graph_safe(self) -> bool:
@@ -61,6 +65,46 @@ class PreNormBlock(Block):
         if self.feed_forward is not None:
             stream.add(self.feed_forward.forward(
                 normed(self.ffn_norm, stream, self.feed_forward), step), m)
+
+
+@register("block", "sandwich")
+class SandwichBlock(PreNormBlock):
+    """Norms in front of the sublayers and behind them: ``x += mixer_post(mixer(mixer_norm(x)))``,
+    then ``x += ffn_post(ff(ffn_norm(x)))``.
+
+    Parameters: those of ``prenorm`` (without ``residual_scale``) and ``mixer_post``, ``ffn_post``
+    (PartSpecs, named in ``names`` like the others).  A sublayer's result is left pending with the
+    norm behind it; one kernel norms it, adds it to the float32 stream and applies the norm that
+    the next sublayer reads through."""
+
+    _SLOTS = (("mixer_norm", "norm"), ("mixer", "mixer"), ("mixer_post", "norm"),
+              ("ffn_norm", "norm"), ("feed_forward", "feed_forward"), ("ffn_post", "norm"))
+
+    @classmethod
+    def _slots(cls, params: Dict[str, Any]):
+        return cls._SLOTS if params.get("feed_forward") is not None else cls._SLOTS[:3]
+
+    def _take(self, built: Dict[str, Any]) -> None:
+        super()._take(built)
+        self.mixer_post, self.ffn_post = built["mixer_post"], built.get("ffn_post")
+
+    def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
+        super().__init__(params, prefix, ctx)
+        if self.residual_scale != 1.0:
+            raise ValueError("block 'sandwich': the norms behind the sublayers scale the results")
+
+    @property
+    def graph_safe(self) -> bool:
+        return all(p.graph_safe for p in (self.mixer_norm, self.mixer, self.mixer_post,
+                                          self.ffn_norm, self.feed_forward, self.ffn_post)
+                   if p is not None)
+
+    def forward(self, stream: ResidualStream, step: Any, binding: CacheBinding) -> None:
+        stream.add(self.mixer.forward(normed(self.mixer_norm, stream, self.mixer), step, binding),
+                   norm=self.mixer_post)
+        if self.feed_forward is not None:
+            stream.add(self.feed_forward.forward(
+                normed(self.ffn_norm, stream, self.feed_forward), step), norm=self.ffn_post)
 
 
 @register("block", "hyper")

@@ -13,8 +13,9 @@ the matrix-core kernel loads it as values.)
 
 Options, each a parameter: a rotated part (``rot_dim`` 0: none), a sliding window, a learned
 sink per head in the softmax's denominator, a sigmoid gate on the heads' outputs (its own
-projection of the mixer's input), and reading the latents that an earlier run has cached
-instead of making one's own (the run's binding then does not write, and the mixer has no
+projection of the mixer's input), queries that go through a normed latent of their own
+(``q = Wuq norm(Wdq h)``), a rotation of neighbouring entries (the position part's), and reading
+the latents that an earlier run has cached instead of making one's own (the run's binding then does not write, and the mixer has no
 down projection).  Scores, softmax, the latent's norm and the rotation are float32."""
 from __future__ import annotations
 
@@ -35,9 +36,11 @@ class LatentAttention(Mixer):
     norm), ``window`` (None: every earlier position), ``cache_window`` (what the cache keeps:
     the widest window among the runs that read it; None: everything), ``sink`` (bool),
     ``gate`` (bool), ``own_latent`` (False: reads another run's cache), ``position`` (a
-    PartSpec, needed with ``rot_dim``).
+    PartSpec, needed with ``rot_dim``), ``q_rank`` (None: queries straight from the input; needs
+    ``own_latent``).
 
-    Tensors under the prefix: ``q`` (heads * (dim + rot_dim), W); ``dkv`` (kv_rank + rot_dim,
+    Tensors under the prefix: ``q`` (heads * (dim + rot_dim), W), or with ``q_rank`` ``dq`` (q_rank,
+    W), ``dq.norm`` (q_rank) and ``uq`` (heads * (dim + rot_dim), q_rank); ``dkv`` (kv_rank + rot_dim,
     W) and ``dkv.norm`` (kv_rank) with ``own_latent``; ``uk`` (heads * dim, kv_rank), ``uv``
     (heads * vdim, kv_rank); ``sink`` (heads); ``g`` (heads * vdim, W); ``o`` (W, heads *
     vdim)."""
@@ -48,7 +51,13 @@ class LatentAttention(Mixer):
     def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
         W, H, d, r = (params[k] for k in ("hidden_size", "num_heads", "head_dim", "rot_dim"))
         dv, R = params["value_dim"], params["kv_rank"]
-        out = [TensorSpec(join(prefix, "q"), (H * (d + r), W))]
+        Rq = params.get("q_rank")
+        if Rq:
+            out = [TensorSpec(join(prefix, "dq"), (Rq, W)),
+                   TensorSpec(join(prefix, "dq.norm"), (Rq,), init="ones_normal"),
+                   TensorSpec(join(prefix, "uq"), (H * (d + r), Rq))]
+        else:
+            out = [TensorSpec(join(prefix, "q"), (H * (d + r), W))]
         if params.get("own_latent", True):
             out += [TensorSpec(join(prefix, "dkv"), (R + r, W)),
                     TensorSpec(join(prefix, "dkv.norm"), (R,), init="ones_normal")]
@@ -78,9 +87,28 @@ class LatentAttention(Mixer):
         self.act_dtype = ctx.act_dtype
         take = lambda n: ctx.take(join(prefix, n))
         H, d, dv, R = self.heads, self.dim, self.vdim, self.rank
-        self.w_q = take("q")
+        self.q_rank = int(params.get("q_rank") or 0)
+        if self.q_rank and not self.own_latent:
+            raise ValueError("latent_attention: a latent for the queries is built for mixers with a "
+                             "latent of their own for keys and values")
+        if self.q_rank:
+            # both down projections read the same input: one product, the queries' rows in front
+            # (padded so that the rows behind them start on 16-byte boundaries)
+            dq, dkv = ctx.weights.pop(join(prefix, "dq")), ctx.weights.pop(join(prefix, "dkv"))
+            if dq.dtype != dkv.dtype:
+                dq, dkv = dq.to(torch.float32), dkv.to(torch.float32)
+            pad, tail = -dq.shape[0] % 8, -dkv.shape[0] % 8
+            self.kv_at = dq.shape[0] + pad
+            self.w_down = torch.cat([dq, dq.new_zeros((pad, dq.shape[1])), dkv,
+                                     dkv.new_zeros((tail, dkv.shape[1]))], dim=0).contiguous()
+            del dq, dkv
+            self.q_norm = take("dq.norm").to(torch.float32).contiguous()
+            self.w_q = take("uq")
+        else:
+            self.w_q = take("q")
+            if self.own_latent:
+                self.w_dkv = take("dkv")
         if self.own_latent:
-            self.w_dkv = take("dkv")
             self.norm = take("dkv.norm").to(torch.float32).contiguous()
         # per head, as (out, in): Uk^T (rank x dim) in front of the attention, Uv (vdim x rank)
         # behind it
@@ -115,17 +143,35 @@ class LatentAttention(Mixer):
         if self.position is not None and step.max_context > self.position.max_positions:
             raise ValueError(f"sequence of {step.max_context} positions exceeds max_seq_len "
                              f"{self.position.max_positions}")
-        q = ops.linear(x, self.w_q, self.act_dtype)                    # (T, H * (d + r))
+        cos = self.position.cos if self.rot_dims else None
+        sin = self.position.sin if self.rot_dims else None
+        pairs = bool(getattr(self.position, "interleaved", False))
         q_lat = torch.empty((T, H * (R + r)), dtype=self.act_dtype, device=x.device)
-        ops.head_linear(q, self.w_uk_t, d + r, out=q_lat, out_head=R + r)
-        writes = binding.writes and self.own_latent
-        if writes or r:
-            down = ops.linear_f32(x, self.w_dkv) if writes else None
-            cos = self.position.cos if self.rot_dims else None
-            sin = self.position.sin if self.rot_dims else None
-            ops.latent_write(down, self.norm if writes else None, self.eps, R, r, self.rot_dims,
-                             cos, sin, step.positions, group.slots if writes else None, pages,
-                             q if r else None, d + r, q_lat if r else None, H, pages_t)
+        if self.q_rank:
+            # one product for both latents, one kernel that norms both and writes the cache; then
+            # the queries from theirs
+            down = ops.linear_f32(x, self.w_down)
+            cq = torch.empty((T, self.q_rank), dtype=self.act_dtype, device=x.device)
+            kv = down[:, self.kv_at:self.kv_at + R + r]
+            ops.latent_write(kv if binding.writes else None, self.norm, self.eps, R, r,
+                             self.rot_dims, cos, sin, step.positions, group.slots, pages, None,
+                             d + r, None, H, pages_t, pairs,
+                             (down[:, :self.q_rank], self.q_norm, cq))
+            q = ops.linear(cq, self.w_q, self.act_dtype)               # (T, H * (d + r))
+            ops.head_linear(q, self.w_uk_t, d + r, out=q_lat, out_head=R + r)
+            if r:
+                ops.latent_write(None, None, self.eps, R, r, self.rot_dims, cos, sin,
+                                 step.positions, None, pages, q, d + r, q_lat, H, None, pairs)
+        else:
+            q = ops.linear(x, self.w_q, self.act_dtype)                # (T, H * (d + r))
+            ops.head_linear(q, self.w_uk_t, d + r, out=q_lat, out_head=R + r)
+            writes = binding.writes and self.own_latent
+            if writes or r:
+                down = ops.linear_f32(x, self.w_dkv) if writes else None
+                ops.latent_write(down, self.norm if writes else None, self.eps, R, r,
+                                 self.rot_dims, cos, sin, step.positions,
+                                 group.slots if writes else None, pages, q if r else None, d + r,
+                                 q_lat if r else None, H, pages_t, pairs)
         mixed = ops.latent_attention(q_lat, pages, group.block_tables, step.seq_of_token,
                                      step.positions, H, R, self.scale, self.window, self.sink,
                                      pages_t, step.cu_seqlens, step.num_seqs)

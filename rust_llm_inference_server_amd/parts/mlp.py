@@ -13,28 +13,35 @@ from .base import BuildContext, FeedForward, TensorSpec, join, project, register
 
 @register("feed_forward", "swiglu")
 class SwiGLU(FeedForward):
-    """Parameters: ``hidden_size``, ``intermediate_size``."""
+    """Parameters: ``hidden_size``, ``intermediate_size``; optional ``names`` (the tensors of gate,
+    up and down under the prefix; default ``gate_proj.weight`` and so on)."""
 
     graph_safe = True
 
     takes_normed_input = True
 
     @classmethod
+    def _names(cls, params: Dict[str, Any], prefix: str) -> Dict[str, str]:
+        names = {**{n: f"{n}_proj.weight" for n in ("gate", "up", "down")},
+                 **(params.get("names") or {})}
+        return {k: join(prefix, v) for k, v in names.items()}
+
+    @classmethod
     def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
         H, I = params["hidden_size"], params["intermediate_size"]
-        return [TensorSpec(join(prefix, "gate_proj.weight"), (I, H)),
-                TensorSpec(join(prefix, "up_proj.weight"), (I, H)),
-                TensorSpec(join(prefix, "down_proj.weight"), (H, I))]
+        n = cls._names(params, prefix)
+        return [TensorSpec(n["gate"], (I, H)), TensorSpec(n["up"], (I, H)),
+                TensorSpec(n["down"], (H, I))]
 
     def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
         super().__init__(params, prefix, ctx)
-        gate = ctx.weights.pop(join(prefix, "gate_proj.weight"))
-        up = ctx.weights.pop(join(prefix, "up_proj.weight"))
+        n = self._names(params, prefix)
+        gate, up = ctx.weights.pop(n["gate"]), ctx.weights.pop(n["up"])
         if gate.dtype != up.dtype:
             gate, up = gate.to(torch.float32), up.to(torch.float32)
         self.w_gate_up = torch.cat([gate, up], dim=0).contiguous()
         del gate, up
-        self.w_down = ctx.take(join(prefix, "down_proj.weight"))
+        self.w_down = ctx.take(n["down"])
         self.act_dtype = ctx.act_dtype
 
     def forward(self, x: Any, step: Any) -> torch.Tensor:
@@ -219,10 +226,12 @@ class RoutedSwiGLU(FeedForward):
     score), ``renormalise`` (the chosen experts' weights are divided by their sum + 1e-20),
     ``correction`` (False: the router has no correction tensor), ``limit`` and ``alpha`` (with a
     limit the units are of the bounded kind, ``g sigmoid(alpha g) (u + 1)`` with
-    ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``).
+    ``g = min(gate, limit)``, ``u = clamp(up, -limit, limit)``), ``identity`` (so many further
+    experts stand behind the others in the router; they have no tensors and hand back the input
+    they were given, times their weight).
 
-    Tensors under the prefix: ``router`` (experts, W), ``correction`` (experts: added to the
-    sigmoid scores for the choice only), ``e<i>.gate|up`` (F, W), ``e<i>.down`` (W, F),
+    Tensors under the prefix: ``router`` (experts + identity, W), ``correction`` (experts + identity: added
+    to the scores for the choice only), ``e<i>.gate|up`` (F, W), ``e<i>.down`` (W, F),
     ``shared.gate|up|down``.  Router logits, scores and the choice are float32.  A block that
     hands over the float32 residual rows and the layer norm in front (``wants_residual``) lets
     the router decide on the unrounded normalised input: the logits then come from one kernel
@@ -235,14 +244,15 @@ class RoutedSwiGLU(FeedForward):
     @classmethod
     def tensor_specs(cls, params: Dict[str, Any], prefix: str) -> List[TensorSpec]:
         W, F, E = params["hidden_size"], params["expert_size"], params["experts"]
+        all_experts = E + int(params.get("identity") or 0)
         out: List[TensorSpec] = []
         for e in range(E):
             out += [TensorSpec(join(prefix, f"e{e}.gate"), (F, W)),
                     TensorSpec(join(prefix, f"e{e}.up"), (F, W)),
                     TensorSpec(join(prefix, f"e{e}.down"), (W, F))]
-        out += [TensorSpec(join(prefix, "router"), (E, W), std=0.5)]
+        out += [TensorSpec(join(prefix, "router"), (all_experts, W), std=0.5)]
         if params.get("correction", True):
-            out += [TensorSpec(join(prefix, "correction"), (E,), std=0.1)]
+            out += [TensorSpec(join(prefix, "correction"), (all_experts,), std=0.1)]
         S = params.get("shared_size")
         if S:
             out += [TensorSpec(join(prefix, "shared.gate"), (S, W)),
@@ -253,6 +263,7 @@ class RoutedSwiGLU(FeedForward):
     def __init__(self, params: Dict[str, Any], prefix: str, ctx: BuildContext):
         super().__init__(params, prefix, ctx)
         E = self.experts = int(params["experts"])
+        self.identity = int(params.get("identity") or 0)
         self.top, self.groups, self.keep = int(params["top"]), int(params["groups"]), int(params["keep"])
         self.scale = float(params.get("scale", 1.0))
         self.scores = params.get("scores", "sigmoid")
@@ -265,9 +276,12 @@ class RoutedSwiGLU(FeedForward):
                              f"'{self.group_score}'")
         if self.limit < 0:
             raise ValueError(f"routed_swiglu: limit {self.limit} must be positive")
-        if E % self.groups or not 1 <= self.keep <= self.groups \
-                or not 1 <= self.top <= self.keep * (E // self.groups):
-            raise ValueError(f"routed_swiglu: {E} experts in {self.groups} groups, {self.keep} "
+        every = E + self.identity
+        if E < 1 or self.identity < 0:
+            raise ValueError(f"routed_swiglu: {E} experts and {self.identity} identity experts")
+        if every % self.groups or not 1 <= self.keep <= self.groups \
+                or not 1 <= self.top <= self.keep * (every // self.groups):
+            raise ValueError(f"routed_swiglu: {every} experts in {self.groups} groups, {self.keep} "
                              f"kept, {self.top} chosen do not fit")
         pop = lambda n: ctx.weights.pop(join(prefix, n))
         self.act_dtype = ctx.act_dtype
@@ -304,7 +318,7 @@ class RoutedSwiGLU(FeedForward):
             shared = ops.linear(ops.linear_swiglu(x, self.w_shared_gate_up), self.w_shared_down,
                                 self.act_dtype)
         return ops.routed_units(x, self.w_gate_up, self.w_down, chosen, weights, shared,
-                                limit=self.limit, alpha=self.alpha)
+                                limit=self.limit, alpha=self.alpha, identity=self.identity > 0)
 
 
 @register("feed_forward", "routed_mlp")

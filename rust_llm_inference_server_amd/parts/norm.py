@@ -53,6 +53,13 @@ class RMSNorm(Norm):
     def forward(self, stream: ResidualStream) -> torch.Tensor:
         if stream.lanes is not None:
             return stream.lanes.normed(self.weight, self.eps, self.out_dtype)
+        behind = stream.pending_norm
+        if isinstance(behind, RMSNorm) and behind.weight.dtype == self.weight.dtype:
+            # the norm that stands behind the sublayer in front, the sum and this norm in one pass
+            delta = stream.take_raw()
+            return ops.norm_join(stream.x, delta, behind.weight, behind.eps, self.out_dtype,
+                                 round_parts=stream.round_parts, next_weight=self.weight,
+                                 next_eps=self.eps)
         delta, scale = stream.take_delta()
         return ops.add_rmsnorm(stream.x, delta, self.weight, self.eps, self.out_dtype,
                                round_parts=stream.round_parts, delta_scale=scale)
@@ -74,6 +81,8 @@ class RMSNorm(Norm):
         if self.out_dtype != torch.bfloat16 or stream.lanes is not None:
             return None
         if stream.pending_norm is not None:
+            if rows is None:
+                return None         # ``forward`` takes both norms in one pass
             stream.flush()
         if stream.pending is not None and stream.pending_scale != 1.0:
             if rows is not None:

@@ -36,10 +36,14 @@ def linear_geglu(x, w_gate_up):
     return geglu(linear(x, w_gate_up, x.dtype))
 
 
-def norm_join(resid, y, weight, eps, out_dtype=None, round_parts=False):
+def norm_join(resid, y, weight, eps, out_dtype=None, round_parts=False, next_weight=None,
+              next_eps=0.0):
     if y is not None:
         y = (y.sum(0) if y.dim() == 3 else y).float()
         resid += y / torch.sqrt((y * y).mean(-1, keepdim=True) + eps) * weight.float()
+    if next_weight is not None:
+        ms = (resid * resid).mean(-1, keepdim=True)
+        return (resid / torch.sqrt(ms + next_eps) * next_weight.float()).to(out_dtype)
     return None if out_dtype is None else resid.to(out_dtype)
 
 
@@ -302,11 +306,16 @@ def head_linear(x, w, x_head, out=None, out_head=None, out_dtype=None):
     return out
 
 
-def _turned(v, pos, cos, sin, dims):
+def _turned(v, pos, cos, sin, dims, interleaved=False):
     half = dims // 2
     c, s = cos[pos.long()], sin[pos.long()]
     while c.dim() < v.dim():
         c, s = c.unsqueeze(1), s.unsqueeze(1)
+    if interleaved:
+        out = v.clone()
+        a, b = v[..., 0:dims:2], v[..., 1:dims:2]
+        out[..., 0:dims:2], out[..., 1:dims:2] = a * c - b * s, b * c + a * s
+        return out
     a, b = v[..., :half], v[..., half:dims]
     return torch.cat([a * c - b * s, b * c + a * s, v[..., dims:]], dim=-1)
 
@@ -316,22 +325,26 @@ def latent_mfma_ok(dtype, rank, row, page_size=16):
 
 
 def latent_write(x, weight, eps, rank, rot_width, rot_dims, cos, sin, positions, slots, pages, q,
-                 q_head, q_out, heads, pages_t=None):
+                 q_head, q_out, heads, pages_t=None, interleaved=False, query_latent=None):
     D = rank + rot_width
     if x is not None:
         lat = x[:, :rank]
         row = lat / torch.sqrt((lat * lat).mean(-1, keepdim=True) + eps) * weight
         if rot_width:
             kr = x[:, rank:D]
-            row = torch.cat([row, _turned(kr, positions, cos, sin, rot_dims) if rot_dims else kr], -1)
+            row = torch.cat([row, _turned(kr, positions, cos, sin, rot_dims, interleaved)
+                             if rot_dims else kr], -1)
         ps = pages.shape[1]
         for t in range(x.shape[0]):
             pages[int(slots[t]) // ps, int(slots[t]) % ps] = row[t].to(pages.dtype)
-    if rot_width:
+    if query_latent is not None:
+        cq, w, out = query_latent
+        out.copy_((cq / torch.sqrt((cq * cq).mean(-1, keepdim=True) + eps) * w).to(out.dtype))
+    if rot_width and q is not None:
         T = q.shape[0]
         qr = q.float().reshape(T, heads, q_head)[..., q_head - rot_width:]
         if rot_dims:
-            qr = _turned(qr, positions, cos, sin, rot_dims)
+            qr = _turned(qr, positions, cos, sin, rot_dims, interleaved)
         q_out.reshape(T, heads, D)[..., rank:] = qr.to(q_out.dtype)
 
 
@@ -386,12 +399,15 @@ def route(logits, correction, groups, keep, top, scale, scores="sigmoid", group_
 
 
 def routed_units(x, w_gate_up, w_down, chosen, weights, addend=None, limit=0.0, alpha=1.0,
-                 plain=False):
+                 plain=False, identity=False):
     T, W = x.shape
     F = w_gate_up.shape[1] // 2
     out = torch.zeros(T, W)
     for t in range(T):
         for e, wt in zip(chosen[t].tolist(), weights[t].tolist()):
+            if identity and e >= w_gate_up.shape[0]:
+                out[t] += wt * x[t].float()
+                continue
             gu = w_gate_up[e].float() @ x[t].float()
             if plain:
                 hidden = (gu.clamp(min=0.0) ** 2).to(x.dtype).float()
@@ -532,6 +548,22 @@ def rope_kv_write(qkv, num_heads, num_kv_heads, head_dim, cos, sin, positions, s
             v_pages[page, :, :, off] = v[t].to(v_pages.dtype)
 
 
+def norm_rope_kv_write(qkv, num_heads, num_kv_heads, head_dim, real_dim, eps, cos, sin, positions,
+                       slots, k_pages, v_pages, page_size, write_kv=True, interleaved=False):
+    T, nh, nkv, d = qkv.shape[0], num_heads, num_kv_heads, head_dim
+    x = qkv.float().reshape(T, nh + 2 * nkv, d).clone()
+    qk = x[:, :nh + nkv]
+    if cos is not None:
+        qk = _turned(qk, positions, cos, sin, 2 * cos.shape[1], interleaved)
+    qk = qk / torch.sqrt((qk * qk).sum(-1, keepdim=True) / real_dim + eps)
+    qkv[:, :nh * d] = qk[:, :nh].reshape(T, nh * d).to(qkv.dtype)
+    if write_kv:
+        for t in range(T):
+            page, off = int(slots[t]) // page_size, int(slots[t]) % page_size
+            k_pages[page, :, off, :] = qk[t, nh:].to(k_pages.dtype)
+            v_pages[page, :, :, off] = x[t, nh + nkv:].to(v_pages.dtype)
+
+
 def copy_pages(pages, src, dst):
     for s, d in zip(src.tolist(), dst.tolist()):
         pages[:, d] = pages[:, s]
@@ -622,7 +654,8 @@ def install(monkeypatch) -> None:
     import rust_llm_inference_server_amd.ops as ops
     import rust_llm_inference_server_amd.engine.runner as runner
     for name in ("embed", "add_residual", "add_rmsnorm", "swiglu", "linear", "linear_swiglu",
-                 "pending_linear", "can_fuse_norm_linear", "rope_kv_write", "rope_attention",
+                 "pending_linear", "can_fuse_norm_linear", "rope_kv_write", "norm_rope_kv_write",
+                 "rope_attention",
                  "copy_pages", "attention_planner", "paged_attention", "sample_rows",
                  "clamped_glu", "weighted_sum", "linear_f32", "soft_cap_", "shift_mix", "tail_update",
                  "causal_conv", "delta_scan", "decay_scan", "head_norm_gate", "selective_scan",
