@@ -59,7 +59,13 @@ beside its closest kin.
 ``--design ralitar`` times the Ralitar design (norms behind the sublayers, a table of token pairs,
 a token input per layer; of every four layers two are the delta rule with a decay per key channel,
 one is a gated linear recurrence and one attention inside chunks of 1,024); its closest kin is
-Gipotar: ``--design gipotar,ralitar``."""
+Gipotar: ``--design gipotar,ralitar``.
+``--design pozelix`` times the Pozelix design (norms on both sides of the sublayers; a stretch of two
+layers runs three times a step, as many layer runs as the preset has layers; attention over a
+cached latent with queries from a latent of their own beside attention in a window of 1,024, with
+head norms and a gate per head; feed-forwards that alternate between a SwiGLU unit and a routed
+mixture with identity experts).  Its closest kin are Bekunex and Pamolix: ``--design
+bekunex,pamolix,pozelix``."""
 import argparse
 import copy
 import json
@@ -343,15 +349,57 @@ def ralitar_like(cfg: dict) -> dict:
             "layers": [copy.deepcopy(order[i % 4]) for i in range(cfg["num_hidden_layers"])]}
 
 
+def pozelix_like(cfg: dict) -> dict:
+    """A Pozelix configuration at the sizes of a Llama preset: the same width, vocabulary, heads and
+    head size, and as many layer runs as the preset has layers: four layers fewer, of which two in
+    the middle run three times.  Layers alternate between attention over a cached latent (latent of
+    512, queries from a latent of three quarters of the width, a rotated part of 64 stretched by 4)
+    and attention in a window of 1,024; every second pair of layers has the preset's feed-forward,
+    the others a mixture of 32 units of a quarter of its width beside eight identity experts, of
+    which a token takes five (four units and one identity on average): as many active feed-forward
+    weights per token as the preset has."""
+    W, d, H = cfg["hidden_size"], cfg["head_dim"], cfg["num_attention_heads"]
+    ff = cfg["intermediate_size"]
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": ff // 4},
+           "router": {"experts": 32, "identity": 8, "top": 5}}
+    latent = {"type": "latent_attention", "mixer": {
+        "heads": H, "dim": d, "rot_dim": 64, "vdim": d, "kv_rank": 512, "q_rank": W * 3 // 4,
+        "scale": (d + 64) ** -0.5,
+        "rot": {"dims": 64, "base": cfg["rope_theta"],
+                "scaling": {"factor": 4.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}}
+    windowed = {"type": "attention", "mixer": {
+        "heads": H, "kv_heads": cfg["num_key_value_heads"], "dim": d, "vdim": d,
+        "scale": d ** -0.5, "mask": {"size": 1024}, "rot": {"dims": d, "base": cfg["rope_theta"]}}}
+    runs = cfg["num_hidden_layers"]
+    n = runs - 4 if runs > 6 else runs
+    layers = [dict(copy.deepcopy(latent if i % 2 == 0 else windowed),
+                   mlp=copy.deepcopy(dense if i // 2 % 2 == 0 else moe)) for i in range(n)]
+    out = {"architecture": "Pozelix", "vocab": cfg["vocab_size"], "width": W,
+           "norm": {"eps": 1e-6}, "layers": layers}
+    if n < runs:
+        a = n // 2 // 2 * 2 + 1           # a windowed layer and a latent one, one of either kind of mlp
+        out["loop"] = {"start": a, "stop": a + 2, "times": 3}
+    return out
+
+
 def step_bytes_of(model, batch: int, mean_context: float) -> float:
     """What a decode step of any model has to move: every tensor its parts hold once (the
-    embedding table only where the head shares it), each live request's cached positions, and
-    its state slot read and written."""
-    seen, total = set(), 0
-    for t in model._tensors():
-        if t.data_ptr() not in seen:
-            seen.add(t.data_ptr())
-            total += t.numel() * t.element_size()
+    embedding table only where the head shares it; a layer that runs several times, once per
+    run), each live request's cached positions, and its state slot read and written."""
+    def tensors_bytes(tensors, seen):
+        total = 0
+        for t in tensors:
+            if t.data_ptr() not in seen:
+                seen.add(t.data_ptr())
+                total += t.numel() * t.element_size()
+        return total
+
+    total = tensors_bytes(model._tensors(), set())
+    for i, layer in enumerate(model.layers):
+        again = sum(r.layer == i for r in model.runs) - 1
+        if again > 0:
+            total += again * tensors_bytes(model._tensors([layer]), set())
     table = model.embedding.weight
     if model.head.weight.data_ptr() != table.data_ptr():
         total -= table.numel() * table.element_size()
@@ -374,13 +422,14 @@ def routed_idle_bytes(model, batch: int) -> float:
     of which every token takes ``top`` at random, E (1 - 1/E)^(batch top) of them stay idle on
     average."""
     idle = 0.0
-    for layer in model.layers:
-        ff = getattr(layer, "feed_forward", None)
+    for run in model.runs:
+        ff = getattr(model.layers[run.layer], "feed_forward", None)
         if ff is not None and hasattr(ff, "experts"):
             E = ff.experts
             up = ff.w_gate_up if hasattr(ff, "w_gate_up") else ff.w_up
             per_expert = (up.numel() + ff.w_down.numel()) * ff.w_down.element_size() / E
-            idle += per_expert * E * (1.0 - 1.0 / E) ** (batch * ff.top)
+            every = E + getattr(ff, "identity", 0)
+            idle += per_expert * E * (1.0 - 1.0 / every) ** (batch * ff.top)
     return idle
 
 
@@ -455,7 +504,7 @@ def compare_designs(args) -> int:
         longest = max(T, args.points_context + new + warm + 16) + 64
         base["max_position_embeddings"] = min(base["max_position_embeddings"], longest)
         like = {"gipotar": gipotar_like, "bekunex": bekunex_like, "lagedra": lagedra_like,
-                "pamolix": pamolix_like, "ralitar": ralitar_like}
+                "pamolix": pamolix_like, "ralitar": ralitar_like, "pozelix": pozelix_like}
         for design, cfg in [("llama", base)] + [(d, like[d](base)) for d in args.design.split(",")]:
             vocab = base["vocab_size"]
             model = random_model(cfg, seed=0, dtype=args.dtype, max_positions=longest)
@@ -517,7 +566,7 @@ def main() -> int:
                     help="time the Gipotar design beside the Llama presets of --sizes instead")
     ap.add_argument("--design", default="gipotar",
                     help="the designs that --designs times beside Llama, with commas between "
-                         "them: gipotar, bekunex, lagedra, pamolix, ralitar")
+                         "them: gipotar, bekunex, lagedra, pamolix, ralitar, pozelix")
     ap.add_argument("--sizes", default="llama-3.2-1b,llama-3.2-3b",
                     help="presets whose sizes the two designs of --designs are built at")
     args = ap.parse_args()

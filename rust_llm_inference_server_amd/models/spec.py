@@ -146,12 +146,12 @@ class Model:
                 seen.add(planner.key())
                 self.step_planners.append(planner)
 
-    def _tensors(self):
-        """Every tensor that a part of the model holds as an attribute (parts within parts
-        included)."""
+    def _tensors(self, parts: Any = None):
+        """Every tensor that a part of the model (or of ``parts``) holds as an attribute (parts
+        within parts included)."""
         from ..parts.base import Part
-        todo, seen = [self.embedding, *self.layers, *self.junctions, self.final_norm,
-                      self.head], set()
+        todo, seen = list(parts if parts is not None else [
+            self.embedding, *self.layers, *self.junctions, self.final_norm, self.head]), set()
         while todo:
             part = todo.pop()
             if id(part) in seen:
