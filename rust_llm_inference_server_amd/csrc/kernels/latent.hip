@@ -11,6 +11,7 @@
 // under a window w, > p - w.  With a sink the softmax's denominator also holds exp(sink[h]):
 // a key with that score (not scaled) and no value.
 #include "common.h"
+#include "kv_write.h"
 #include "tile_mma.h"
 
 #include <math.h>
@@ -215,6 +216,50 @@ __global__ __launch_bounds__(256) void latent_write_kernel(
   }
 }
 
+// The queries' part alone, bfloat16 in pieces of eight: a thread per piece.
+template <bool INTERLEAVED>
+__global__ __launch_bounds__(256) void latent_turn_queries_kernel(
+    const bf16_t* __restrict__ q, long long ldq, int q_head, int q_off, bf16_t* __restrict__ q_out,
+    long long ldo, int o_head, int R, int r, int rot, const float* __restrict__ cos_t,
+    const float* __restrict__ sin_t, const int* __restrict__ positions, int H, unsigned pieces) {
+  const unsigned i = blockIdx.x * 256u + threadIdx.x;
+  if (i >= pieces) return;
+  const unsigned per_head = r / 8, per_tok = H * per_head;
+  const unsigned t = i / per_tok, rest = i - t * per_tok, h = rest / per_head;
+  const int j = (int)(rest - h * per_head) * 8, half = rot / 2;
+  const bf16_t* src = q + (long long)t * ldq + (long long)h * q_head + q_off;
+  float v[8];
+  unpack8(*(const uint4*)(src + j), v);
+  if (j < rot) {
+    const float* cos_r = cos_t + (long long)positions[t] * half;
+    const float* sin_r = sin_t + (long long)positions[t] * half;
+    if constexpr (INTERLEAVED) {
+      float c[4], s[4];
+      *(float4*)c = *(const float4*)(cos_r + j / 2);
+      *(float4*)s = *(const float4*)(sin_r + j / 2);
+#pragma unroll
+      for (int e = 0; e < 4; ++e) {
+        const float u = v[2 * e], w = v[2 * e + 1];
+        v[2 * e] = u * c[e] - w * s[e];
+        v[2 * e + 1] = w * c[e] + u * s[e];
+      }
+    } else {
+      const bool first = j < half;
+      const int a = first ? j : j - half;
+      float w[8], c[8], s[8];
+      unpack8(*(const uint4*)(src + (first ? j + half : j - half)), w);
+#pragma unroll
+      for (int e = 0; e < 8; e += 4) {
+        *(float4*)(c + e) = *(const float4*)(cos_r + a + e);
+        *(float4*)(s + e) = *(const float4*)(sin_r + a + e);
+      }
+#pragma unroll
+      for (int e = 0; e < 8; ++e) v[e] = first ? v[e] * c[e] - w[e] * s[e] : v[e] * c[e] + w[e] * s[e];
+    }
+  }
+  *(uint4*)(q_out + (long long)t * ldo + (long long)h * o_head + R + j) = pack8(v);
+}
+
 RLIS_API int rlis_latent_write(const float* x, long long ldx, const float* weight, float eps,
                                int R, int r, int rot, const float* cos_t, const float* sin_t,
                                const int* positions, const int* slots, void* pages,
@@ -234,6 +279,25 @@ RLIS_API int rlis_latent_write(const float* x, long long ldx, const float* weigh
                "latent_write: the queries' latent needs its rows, its weight and a result");
   if (T == 0 || (!write && !q && !cq)) return 0;
   const LatentQuery lq = {cq, ld_cq, cq_R, cq_weight, cq_out};
+  const long long pieces = q ? (long long)T * H * r / 8 : 0;
+  const auto by8 = [](long long a, long long b, long long c, long long d) {
+    return (a | b | c | d) % 8 == 0;
+  };
+  if (q && !write && !cq && dtype == RLIS_BF16 && by8(ldq, q_head, q_off, r) &&
+      by8(ldo, o_head, R, 0) && rot % (interleaved ? 8 : 16) == 0 && pieces < (1ll << 32) - 256 &&
+      ((uintptr_t)q | (uintptr_t)q_out | (uintptr_t)cos_t | (uintptr_t)sin_t) % 16 == 0) {
+    const unsigned blocks = (unsigned)ceil_div_ll(pieces, 256);
+    if (interleaved)
+      latent_turn_queries_kernel<true><<<blocks, 256, 0, stream>>>(
+          (const bf16_t*)q, ldq, q_head, q_off, (bf16_t*)q_out, ldo, o_head, R, r, rot, cos_t, sin_t,
+          positions, H, (unsigned)pieces);
+    else
+      latent_turn_queries_kernel<false><<<blocks, 256, 0, stream>>>(
+          (const bf16_t*)q, ldq, q_head, q_off, (bf16_t*)q_out, ldo, o_head, R, r, rot, cos_t, sin_t,
+          positions, H, (unsigned)pieces);
+    RLIS_LAUNCH_CHECK("latent_write");
+    return 0;
+  }
 #define LAUNCH(TX)                                                                            \
   latent_write_kernel<TX><<<dim3(T, cq ? 2 : 1), 256, 0, stream>>>(                           \
       x, ldx, weight, eps, R, r, rot, cos_t, sin_t, positions, slots, (TX*)pages,             \

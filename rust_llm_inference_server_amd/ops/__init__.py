@@ -1101,11 +1101,12 @@ def norm_rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, hea
                        sin: Optional[torch.Tensor], positions: torch.Tensor,
                        slots: Optional[torch.Tensor], k_pages: Optional[torch.Tensor],
                        v_pages: Optional[torch.Tensor], page_size: int, write_kv: bool = True,
-                       interleaved: bool = False) -> None:
+                       interleaved: bool = False, keys_in_place: bool = False) -> None:
     """``rope_kv_write`` for queries and keys that are divided by their root mean square behind
     the rotation: every q and k head of ``qkv (T, (nh + 2 nkv) d)`` is rotated and then divided by
     ``sqrt(mean(head^2) + eps)``, the mean over its first ``real_dim`` numbers (the others are
-    zero padding).  q in place; with ``write_kv`` k and v go to the pages."""
+    zero padding).  q in place; with ``write_kv`` k and v go to the pages, with ``keys_in_place``
+    k stays in its row and nothing is written (the attention kernel does that)."""
     stride = _rows_contig(qkv, "qkv")
     T, nh, nkv, d = qkv.shape[0], int(num_heads), int(num_kv_heads), int(head_dim)
     if qkv.shape[1] != (nh + 2 * nkv) * d:
@@ -1119,6 +1120,8 @@ def norm_rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, hea
             raise KernelError("norm_rope_kv_write: cos and sin must match and be contiguous")
         rot, cos_ptr, sin_ptr = 2 * cos.shape[1], cos.data_ptr(), sin.data_ptr()
     kp = vp = sp = None
+    if write_kv and keys_in_place:
+        raise KernelError("norm_rope_kv_write: keys go to the pages or stay in place, not both")
     if write_kv:
         if k_pages is None or v_pages is None or slots is None:
             raise KernelError("norm_rope_kv_write: a cache write needs pages and slots")
@@ -1132,7 +1135,7 @@ def norm_rope_kv_write(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, hea
     lib.call("rlis_norm_rope_kv_write", qkv.data_ptr(), _dt(qkv), stride, nh * d, (nh + nkv) * d, T,
              nh, nkv, d, int(real_dim), rot, float(eps), cos_ptr, sin_ptr,
              _i32(positions, "positions", T), sp, kp, vp, page_size, int(bool(interleaved)),
-             int(bool(write_kv)), lib.stream_ptr())
+             2 if keys_in_place else int(bool(write_kv)), lib.stream_ptr())
 
 
 def copy_pages(pages: torch.Tensor, src: torch.Tensor, dst: torch.Tensor) -> None:
@@ -1281,6 +1284,34 @@ def rope_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_di
     return paged_attention(qkv, nh, nkv, d, k_pages, v_pages, page_size, block_tables, step,
                            scale, window, plan=plan, bias_slopes=bias_slopes, counters=counters,
                            **more)
+
+
+def norm_rope_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,
+                        real_dim: int, eps: float, cos: Optional[torch.Tensor],
+                        sin: Optional[torch.Tensor], positions: torch.Tensor,
+                        slots: Optional[torch.Tensor], k_pages: torch.Tensor,
+                        v_pages: torch.Tensor, page_size: int, block_tables: torch.Tensor, step,
+                        scale: float, window: Optional[int] = None, write_kv: bool = True,
+                        interleaved: bool = False, plan: Optional[StepPlan] = None,
+                        bias_slopes: Optional[torch.Tensor] = None,
+                        counters: Optional[torch.Tensor] = None, **more) -> torch.Tensor:
+    """``norm_rope_kv_write`` followed by ``paged_attention`` (``more``: its other options).  A
+    decode batch that takes the matrix-core decode kernel has its keys normed in their rows, and
+    that kernel writes them and the values to the pages."""
+    nh, nkv, d = num_heads, num_kv_heads, head_dim
+    shaped = more.get("head_scales") is not None or more.get("softcap", 0.0) > 0
+    _, mfma = _attention_kernel(qkv, nh, nkv, d, page_size, step, None, bias_slopes is not None,
+                                shaped, PLAIN_EXTRAS and (more.get("sinks") is not None or bool(
+                                    more.get("keep_first") and window)))
+    fused = mfma and write_kv and FUSE_ROPE_DECODE
+    if fused and slots is None:
+        raise KernelError("norm_rope_attention: a cache write needs slots")
+    norm_rope_kv_write(qkv, nh, nkv, d, real_dim, eps, cos, sin, positions, slots, k_pages, v_pages,
+                       page_size, write_kv=write_kv and not fused, interleaved=interleaved,
+                       keys_in_place=fused)
+    return paged_attention(qkv, nh, nkv, d, k_pages, v_pages, page_size, block_tables, step, scale,
+                           window, plan=plan, bias_slopes=bias_slopes, counters=counters, **more,
+                           rope=(None, None, positions, slots) if fused else None)
 
 
 def paged_attention(qkv: torch.Tensor, num_heads: int, num_kv_heads: int, head_dim: int,

@@ -390,19 +390,15 @@ class PagedAttention(Mixer):
                        ) -> torch.Tensor:
         """Queries and keys normed behind their rotation: one kernel in front of the attention."""
         pos = self.position
-        ops.norm_rope_kv_write(qkv, self.num_heads, self.num_kv_heads, self.head_dim, self.qk_dim,
-                               self.norm_eps, pos.cos, pos.sin, step.positions, group.slots,
-                               binding.k_pages, binding.v_pages, group.page_size,
-                               write_kv=binding.writes,
-                               interleaved=bool(getattr(pos, "interleaved", False)))
-        return ops.paged_attention(qkv, self.num_heads, self.num_kv_heads, self.head_dim,
-                                   binding.k_pages, binding.v_pages, group.page_size,
-                                   group.block_tables, step, self.scale, self.window,
-                                   plan=step.plans.get(self.planner.key()),
-                                   bias_slopes=getattr(pos, "bias_slopes", None),
-                                   counters=binding.counters, head_scales=self.head_scales,
-                                   softcap=self.softcap, sinks=self.sinks,
-                                   keep_first=self.keep_first, chunk=self.chunk)
+        return ops.norm_rope_attention(
+            qkv, self.num_heads, self.num_kv_heads, self.head_dim, self.qk_dim, self.norm_eps,
+            pos.cos, pos.sin, step.positions, group.slots, binding.k_pages, binding.v_pages,
+            group.page_size, group.block_tables, step, self.scale, self.window,
+            write_kv=binding.writes, interleaved=bool(getattr(pos, "interleaved", False)),
+            plan=step.plans.get(self.planner.key()),
+            bias_slopes=getattr(pos, "bias_slopes", None), counters=binding.counters,
+            head_scales=self.head_scales, softcap=self.softcap, sinks=self.sinks,
+            keep_first=self.keep_first, chunk=self.chunk)
 
     def _attend(self, qkv: torch.Tensor, step: Any, binding: CacheBinding, group: Any
                 ) -> torch.Tensor:

@@ -549,7 +549,8 @@ def rope_kv_write(qkv, num_heads, num_kv_heads, head_dim, cos, sin, positions, s
 
 
 def norm_rope_kv_write(qkv, num_heads, num_kv_heads, head_dim, real_dim, eps, cos, sin, positions,
-                       slots, k_pages, v_pages, page_size, write_kv=True, interleaved=False):
+                       slots, k_pages, v_pages, page_size, write_kv=True, interleaved=False,
+                       keys_in_place=False):
     T, nh, nkv, d = qkv.shape[0], num_heads, num_kv_heads, head_dim
     x = qkv.float().reshape(T, nh + 2 * nkv, d).clone()
     qk = x[:, :nh + nkv]
@@ -562,6 +563,16 @@ def norm_rope_kv_write(qkv, num_heads, num_kv_heads, head_dim, real_dim, eps, co
             page, off = int(slots[t]) // page_size, int(slots[t]) % page_size
             k_pages[page, :, off, :] = qk[t, nh:].to(k_pages.dtype)
             v_pages[page, :, :, off] = x[t, nh + nkv:].to(v_pages.dtype)
+
+
+def norm_rope_attention(qkv, num_heads, num_kv_heads, head_dim, real_dim, eps, cos, sin, positions,
+                        slots, k_pages, v_pages, page_size, block_tables, step, scale, window=None,
+                        write_kv=True, interleaved=False, plan=None, bias_slopes=None,
+                        counters=None, **more):
+    norm_rope_kv_write(qkv, num_heads, num_kv_heads, head_dim, real_dim, eps, cos, sin, positions,
+                       slots, k_pages, v_pages, page_size, write_kv, interleaved)
+    return paged_attention(qkv, num_heads, num_kv_heads, head_dim, k_pages, v_pages, page_size,
+                           block_tables, step, scale, window, bias_slopes=bias_slopes, **more)
 
 
 def copy_pages(pages, src, dst):
@@ -655,6 +666,7 @@ def install(monkeypatch) -> None:
     import rust_llm_inference_server_amd.engine.runner as runner
     for name in ("embed", "add_residual", "add_rmsnorm", "swiglu", "linear", "linear_swiglu",
                  "pending_linear", "can_fuse_norm_linear", "rope_kv_write", "norm_rope_kv_write",
+                 "norm_rope_attention",
                  "rope_attention",
                  "copy_pages", "attention_planner", "paged_attention", "sample_rows",
                  "clamped_glu", "weighted_sum", "linear_f32", "soft_cap_", "shift_mix", "tail_update",
