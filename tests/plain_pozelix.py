@@ -113,12 +113,15 @@ def attention(h: torch.Tensor, m: Dict[str, Any], w: Dict[str, torch.Tensor], pr
     """Grouped heads under a sliding window; queries and keys rotated, then divided by their root
     mean square; a gate per head on the result."""
     n, H, G = h.shape[0], m["heads"], m["kv_heads"]
-    q = rms(rotate_halves((h @ w[pre + "q"].T).reshape(n, H, m["dim"]), m["rot"]), eps)
-    k = rms(rotate_halves((h @ w[pre + "k"].T).reshape(n, G, m["dim"]), m["rot"]), eps)
+    q = (h @ w[pre + "q"].T).reshape(n, H, m["dim"])
+    k = (h @ w[pre + "k"].T).reshape(n, G, m["dim"])
+    if m.get("rot"):
+        q, k = rotate_halves(q, m["rot"]), rotate_halves(k, m["rot"])
+    q, k = rms(q, eps), rms(k, eps)
     v = (h @ w[pre + "v"].T).reshape(n, G, m["vdim"])
     of = [i // (H // G) for i in range(H)]
     scores = torch.stack([q[:, i] @ k[:, of[i]].T for i in range(H)]) * m["scale"]
-    out = attend(scores, visible(n, m["mask"]["size"]), v[:, of])
+    out = attend(scores, visible(n, (m.get("mask") or {}).get("size")), v[:, of])
     out = out * torch.sigmoid(h @ w[pre + "g"].T).unsqueeze(-1)
     return out.reshape(n, -1) @ w[pre + "o"].T
 
